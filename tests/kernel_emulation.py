@@ -13,6 +13,8 @@ import math
 
 import torch
 
+from wllm_amd.kernels import ops
+
 
 class EmulatedKernels:
     def __init__(self, precise: bool = False, splits: int = 1):
@@ -626,6 +628,10 @@ class EmulatedKernels:
             a = 0.5 * g * (1.0 + torch.tanh(math.sqrt(2.0 / math.pi) * (g + 0.044715 * g.pow(3))))
         elif activation == "silu":
             a = g * torch.sigmoid(g)
+        elif isinstance(activation, ops.ClampedSwish):
+            c = activation
+            g = torch.clamp(g, max=c.limit)
+            a, u = g * torch.sigmoid(c.slope * g), torch.clamp(u, -c.limit, c.limit) + c.shift
         else:
             raise ValueError(activation)
         out.copy_((a * u).to(out.dtype))

@@ -45,6 +45,23 @@ def _position(rotation) -> PositionSpec:
                         scaling_factor=rotation.scaling_factor)
 
 
+def exponential_memory(width: int, eps: float, m, p: str, output_scale: float = 1.0) -> MatrixMemorySpec:
+    """The mLSTM's matrix memory of the sizes `m` (heads, dim, vdim, gate_cap), its tensors named `p` + ..."""
+    return MatrixMemorySpec(
+        hidden_size=width, num_heads=m.heads, head_dim=m.dim, value_dim=m.vdim, gating="exponential", gate_cap=m.gate_cap,
+        den_eps=DEN_EPS, q_scale=m.dim ** -0.5, norm_eps=eps, norm_weight=p + "norm", gate_activation="sigmoid",
+        output_scale=output_scale, q_weight=p + "q", k_weight=p + "k", v_weight=p + "v", gate_weight=p + "g",
+        o_weight=p + "o", i_weight=p + "i", i_bias=p + "i.b", f_weight=p + "f", f_bias=p + "f.b")
+
+
+def retention_memory(width: int, eps: float, m, p: str) -> MatrixMemorySpec:
+    """Retention of the sizes `m` (heads, dim, vdim, decay, rotation), its tensors named `p` + ..."""
+    return MatrixMemorySpec(
+        hidden_size=width, num_heads=m.heads, head_dim=m.dim, value_dim=m.vdim, gating="decay", decays=m.decay,
+        k_scale=m.dim ** -0.5, position=_position(m.rotation), norm_eps=eps, gate_activation="silu", q_weight=p + "q",
+        k_weight=p + "k", v_weight=p + "v", gate_weight=p + "g", o_weight=p + "o")
+
+
 def lefisun_plan(cfg: LefisunConfig) -> ModelPlan:
     def norm(name: str) -> NormSpec:
         return NormSpec(size=cfg.width, eps=cfg.norm_eps, weight=name, kind="rms")
@@ -61,20 +78,10 @@ def lefisun_plan(cfg: LefisunConfig) -> ModelPlan:
                 q_bias=p + "left.q.b", k_bias=p + "left.k.b", v_bias=p + "left.v.b",
                 q_norm_weight=p + "left.q.norm", k_norm_weight=p + "left.k.norm", band_norm_eps=cfg.norm_eps,
                 bias_before_norm=True, sink=0.0, weights_in_float32=True, output_scale=m.left_scale)
-            right = MatrixMemorySpec(
-                hidden_size=cfg.width, num_heads=r.heads, head_dim=r.dim, value_dim=r.vdim, gating="exponential",
-                gate_cap=r.gate_cap, den_eps=DEN_EPS, q_scale=r.dim ** -0.5, norm_eps=cfg.norm_eps,
-                norm_weight=p + "right.norm", gate_activation="sigmoid", output_scale=m.right_scale,
-                q_weight=p + "right.q", k_weight=p + "right.k", v_weight=p + "right.v", gate_weight=p + "right.g",
-                o_weight=p + "right.o", i_weight=p + "right.i", i_bias=p + "right.i.b", f_weight=p + "right.f",
-                f_bias=p + "right.f.b")
+            right = exponential_memory(cfg.width, cfg.norm_eps, r, p + "right.", output_scale=m.right_scale)
             mixer = SideBySideSpec(left=left, right=right)
         else:
-            mixer = MatrixMemorySpec(
-                hidden_size=cfg.width, num_heads=m.heads, head_dim=m.dim, value_dim=m.vdim, gating="decay",
-                decays=m.decay, k_scale=m.dim ** -0.5, position=_position(m.rotation), norm_eps=cfg.norm_eps,
-                gate_activation="silu", q_weight=p + "q", k_weight=p + "k", v_weight=p + "v", gate_weight=p + "g",
-                o_weight=p + "o")
+            mixer = retention_memory(cfg.width, cfg.norm_eps, m, p)
         q = f"l{i}."
         e = layer.mlp
         feed_forward = None

@@ -162,6 +162,35 @@ __device__ __forceinline__ float activate(float z) {
     return z / (1.f + expf(-z));
 }
 
+// The whole step between a gated feed-forward's two products, as the kernels that make both halves know it: the
+// activations above (activate(gate) * up), and behind them the clamped swish, g sigmoid(slope g) (u + shift) with
+// g = min(gate, limit) and u held within -limit .. limit.  `GateShape` is what the host passes for the latter (the
+// others do not read it).
+constexpr int kGateClampedSwish = kActivations;
+constexpr int kGates = kActivations + 1;
+
+struct GateShape {
+    float limit, slope, shift;
+};
+
+template <int GATE>
+__device__ __forceinline__ float gate_product(float gate, float up, GateShape shape) {
+    static_assert(GATE >= 0 && GATE < kGates, "unknown gate");
+    if (GATE < kActivations) return activate<(GATE < kActivations ? GATE : 0)>(gate) * up;
+    // (comparisons, not fminf/fmaxf: what is not a number stays visible)
+    const float g = gate > shape.limit ? shape.limit : gate;
+    const float u = up > shape.limit ? shape.limit : (up < -shape.limit ? -shape.limit : up);
+    return g / (1.f + expf(-shape.slope * g)) * (u + shape.shift);
+}
+
+// Runs `statement` with the compile-time constant GATE set to the gate's number.
+#define WLLM_BY_GATE(gate, statement)                                                       \
+    switch (gate) {                                                                          \
+        case kActGeluTanh: { constexpr int GATE = kActGeluTanh; statement; } break;          \
+        case kActSilu: { constexpr int GATE = kActSilu; statement; } break;                  \
+        default: { constexpr int GATE = kGateClampedSwish; statement; } break;               \
+    }
+
 // Runs `statement` with the compile-time constant ACT set to the activation's number.
 #define WLLM_BY_ACTIVATION(activation, statement)                                     \
     switch (activation) {                                                              \

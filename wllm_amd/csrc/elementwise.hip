@@ -429,26 +429,26 @@ WLLM_API int wllm_rope_cache_write(void* qkv, int is_bf16, const float* parts, i
 
 // ---- gated activation: out = act(g) * u with g, u the two halves of a row -----------------------
 
-template <typename T, int ACT>
+template <typename T, int GATE>
 __global__ void gated_activation_kernel(const T* __restrict__ gate_up, T* __restrict__ out, long long total,
-                                        int inter, long long out_stride) {
+                                        int inter, long long out_stride, GateShape shape) {
     const long long stride = static_cast<long long>(gridDim.x) * blockDim.x;
     for (long long i = static_cast<long long>(blockIdx.x) * blockDim.x + threadIdx.x; i < total; i += stride) {
         const long long r = i / inter;
         const int c = static_cast<int>(i % inter);
         const float g = to_float(gate_up[r * 2 * inter + c]);
         const float u = to_float(gate_up[r * 2 * inter + inter + c]);
-        out[r * out_stride + c] = from_float<T>(activate<ACT>(g) * u);
+        out[r * out_stride + c] = from_float<T>(gate_product<GATE>(g, u, shape));
     }
 }
 
 // bfloat16 rows whose halves are multiples of 8: eight values per 16-byte load; a workgroup walks one
 // row (blockIdx.y and on), so no thread divides, and the product of the matrix kernel before it is
 // read once
-template <int ACT>
+template <int GATE>
 __global__ void __launch_bounds__(256)
 gated_activation_bf16x8_kernel(const bf16* __restrict__ gate_up, bf16* __restrict__ out, int rows, int inter,
-                               long long out_stride) {
+                               long long out_stride, GateShape shape) {
     const int vecs = inter / 8;
     for (int r = blockIdx.y; r < rows; r += gridDim.y) {
         const bf16* src = gate_up + static_cast<size_t>(r) * 2 * inter;
@@ -462,7 +462,7 @@ gated_activation_bf16x8_kernel(const bf16* __restrict__ gate_up, bf16* __restric
             for (int k = 0; k < 4; ++k) {
                 const float g0 = __uint_as_float(gw[k] << 16), g1 = __uint_as_float(gw[k] & 0xffff0000u);
                 const float u0 = __uint_as_float(uw[k] << 16), u1 = __uint_as_float(uw[k] & 0xffff0000u);
-                ow[k] = pack2_bf16(activate<ACT>(g0) * u0, activate<ACT>(g1) * u1);
+                ow[k] = pack2_bf16(gate_product<GATE>(g0, u0, shape), gate_product<GATE>(g1, u1, shape));
             }
             *reinterpret_cast<uint4*>(dst + v * 8) = make_uint4(ow[0], ow[1], ow[2], ow[3]);
         }
@@ -470,24 +470,24 @@ gated_activation_bf16x8_kernel(const bf16* __restrict__ gate_up, bf16* __restric
 }
 
 // `out_stride`: elements between two rows of out (inter, or more where out is a band of columns of a
-// wider buffer).
-WLLM_API int wllm_gated_activation(const void* gate_up, void* out, int is_bf16, int activation, int n, int inter,
-                                   long long out_stride, hipStream_t stream) {
-    if (activation < 0 || activation >= kActivations || out_stride < inter) return -1;
+// wider buffer).  `gate` is the gate's number; limit, slope and shift are those of the clamped swish.
+WLLM_API int wllm_gated_activation(const void* gate_up, void* out, int is_bf16, int gate, float limit, float slope,
+                                   float shift, int n, int inter, long long out_stride, hipStream_t stream) {
+    if (gate < 0 || gate >= kGates || out_stride < inter) return -1;
+    const GateShape shape{limit, slope, shift};
     const long long total = static_cast<long long>(n) * inter;
     if (is_bf16 && inter % 8 == 0 && out_stride % 8 == 0 && reinterpret_cast<uintptr_t>(out) % 16 == 0) {
         const int vecs = inter / 8;
         const dim3 grid(vecs < 2048 ? (vecs + 255) / 256 : 8, n < 16384 ? n : 16384);
-        WLLM_BY_ACTIVATION(activation, (gated_activation_bf16x8_kernel<ACT><<<grid, 256, 0, stream>>>(
-                                           static_cast<const bf16*>(gate_up), static_cast<bf16*>(out), n, inter,
-                                           out_stride)));
+        WLLM_BY_GATE(gate, (gated_activation_bf16x8_kernel<GATE><<<grid, 256, 0, stream>>>(
+                               static_cast<const bf16*>(gate_up), static_cast<bf16*>(out), n, inter, out_stride, shape)));
         return launch_status();
     }
     long long blocks = (total + 255) / 256;
     if (blocks > 65536) blocks = 65536;
 #define LAUNCH(T)                                                                                                   \
-    WLLM_BY_ACTIVATION(activation, (gated_activation_kernel<T, ACT><<<static_cast<int>(blocks), 256, 0, stream>>>( \
-                                       static_cast<const T*>(gate_up), static_cast<T*>(out), total, inter, out_stride)))
+    WLLM_BY_GATE(gate, (gated_activation_kernel<T, GATE><<<static_cast<int>(blocks), 256, 0, stream>>>(             \
+                           static_cast<const T*>(gate_up), static_cast<T*>(out), total, inter, out_stride, shape)))
     if (is_bf16) { LAUNCH(bf16); } else { LAUNCH(float); }
 #undef LAUNCH
     return launch_status();

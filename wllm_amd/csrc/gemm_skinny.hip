@@ -357,10 +357,10 @@ struct NormOnLoad {
     float eps, offset;
 };
 
-template <int MT, int ACT, bool TILED, int TPW, bool NORM, int XR>
+template <int MT, int GATE, bool TILED, int TPW, bool NORM, int XR>
 __global__ void __launch_bounds__(TPW * 128, MT == 1 ? (NORM && XR > 2 ? 3 : 4) : (MT == 2 ? 3 : 2))
 gemm_skinny_gated_kernel(const bf16* __restrict__ x, NormOnLoad norm, const bf16* __restrict__ w, bf16* __restrict__ out,
-                         int M, int inter, int K, int chunk, int out_stride) {
+                         int M, int inter, int K, int chunk, int out_stride, GateShape shape) {
     extern __shared__ uint4 xs[];                 // two halves of [MT*16][chunk/8 + 1]
     __shared__ float inv_s[16];                   // NORM: a row's rsqrt(mean square + eps)
     const int lane = threadIdx.x % kWave, wave = threadIdx.x / kWave;
@@ -532,7 +532,7 @@ gemm_skinny_gated_kernel(const bf16* __restrict__ x, NormOnLoad norm, const bf16
 #pragma unroll
         for (int v = 0; v < 4; ++v) {
             const float gate = accg[t][v] + red[t * 8 + v], upv = accu[t][v] + red[t * 8 + 4 + v];
-            r[v] = activate<ACT>(gate) * upv;
+            r[v] = gate_product<GATE>(gate, upv, shape);
         }
         bf16* o = out + static_cast<size_t>(m) * out_stride + n;     // out may be a band of columns of a wider buffer
         if (n + 3 < inter && (inter % 4 == 0) && (out_stride % 4 == 0)) {
@@ -546,9 +546,9 @@ gemm_skinny_gated_kernel(const bf16* __restrict__ x, NormOnLoad norm, const bf16
 }
 
 static int gated_launch(const void* x, NormOnLoad norm, bool with_norm, const void* w, int tiled, void* out, int M,
-                        int inter, int K, int activation, int chunk, int out_stride, hipStream_t stream) {
+                        int inter, int K, int gate, GateShape shape, int chunk, int out_stride, hipStream_t stream) {
     if (out_stride < inter) return -1;
-    if (M < 1 || M > 64 || K % 64 != 0 || chunk % 32 != 0 || activation < 0 || activation >= kActivations) return -1;
+    if (M < 1 || M > 64 || K % 64 != 0 || chunk % 32 != 0 || gate < 0 || gate >= kGates) return -1;
     const int mt = (M + 15) / 16;
     if (chunk > K / 2) chunk = K / 2;
     // the norm on load: at most 16 rows, whole chunks of 256 keys
@@ -574,7 +574,7 @@ static int gated_launch(const void* x, NormOnLoad norm, bool with_norm, const vo
         }                                                                                                             \
         gemm_skinny_gated_kernel<MT, A, T, TPW, NORM, XR><<<grid, TPW * 128, smem, stream>>>(                        \
             static_cast<const bf16*>(x), norm, static_cast<const bf16*>(w), static_cast<bf16*>(out), M, inter, K, chunk, \
-            out_stride);                                                                                              \
+            out_stride, shape);                                                                                       \
     } while (0)
 #define LAUNCH_T(MT, A, T, TPW) LAUNCH_K(MT, A, T, TPW, false, 4)
 #define LAUNCH(MT, A)                        \
@@ -596,9 +596,9 @@ static int gated_launch(const void* x, NormOnLoad norm, bool with_norm, const vo
         default: LAUNCH(4, A); break; \
     }
     if (with_norm) {
-        WLLM_BY_ACTIVATION(activation, LAUNCH_N(ACT))
+        WLLM_BY_GATE(gate, LAUNCH_N(GATE))
     } else {
-        WLLM_BY_ACTIVATION(activation, BY_MT(ACT))
+        WLLM_BY_GATE(gate, BY_MT(GATE))
     }
 #undef BY_MT
 #undef LAUNCH_N
@@ -609,12 +609,14 @@ static int gated_launch(const void* x, NormOnLoad norm, bool with_norm, const vo
 }
 
 // `out_stride`: elements between two rows of out (inter, or more where out is a band of columns of a
-// wider buffer; the band then begins at a multiple of 8 bytes).
+// wider buffer; the band then begins at a multiple of 8 bytes).  `gate` is the gate's number; limit, slope and shift
+// are those of the clamped swish.
 WLLM_API int wllm_gemm_skinny_gated(const void* x, const void* w, int tiled, void* out, int M, int inter, int K,
-                                    int activation, int chunk, int out_stride, hipStream_t stream) {
+                                    int gate, float limit, float slope, float shift, int chunk, int out_stride,
+                                    hipStream_t stream) {
     if (reinterpret_cast<uintptr_t>(out) % 8 != 0) return -1;
-    return gated_launch(x, NormOnLoad{nullptr, nullptr, nullptr, 0, 0.f, 0.f}, false, w, tiled, out, M, inter, K, activation,
-                        chunk, out_stride, stream);
+    return gated_launch(x, NormOnLoad{nullptr, nullptr, nullptr, 0, 0.f, 0.f}, false, w, tiled, out, M, inter, K, gate,
+                        GateShape{limit, slope, shift}, chunk, out_stride, stream);
 }
 
 // The same product with the RMS norm of the residual stream folded into the load of x: at most 16
@@ -622,8 +624,8 @@ WLLM_API int wllm_gemm_skinny_gated(const void* x, const void* w, int tiled, voi
 // squares of the row of `residual`.  Returns -1 for sizes it does not take.
 WLLM_API int wllm_gemm_skinny_gated_norm(const float* residual, const float* sumsq, int sumsq_cols, const float* norm_weight,
                                          float eps, float offset, const void* w, int tiled, void* out, int M, int inter,
-                                         int K, int activation, hipStream_t stream) {
+                                         int K, int gate, float limit, float slope, float shift, hipStream_t stream) {
     if (M > 16 || sumsq_cols < 1) return -1;
     return gated_launch(nullptr, NormOnLoad{residual, sumsq, norm_weight, sumsq_cols, eps, offset}, true, w, tiled, out, M,
-                        inter, K, activation, 256, inter, stream);
+                        inter, K, gate, GateShape{limit, slope, shift}, 256, inter, stream);
 }

@@ -50,7 +50,7 @@ static __device__ __forceinline__ void load_to_shared(const void* base, uint32_t
 }
 
 
-// GATED: 0 plain, 1 + the activation's number for the gated product.  N is the number of rows of w (plain) or of gate rows (gated).
+// GATED: 0 plain, 1 + the gate's number for the gated product.  N is the number of rows of w (plain) or of gate rows (gated).
 // (Tiles of 256 rows of x with eight wavefronts were no faster: the rate is set by the reads of
 // fragments from shared memory, which take as long as the products they feed.)
 // STAGES: how many stages' tiles shared memory holds.  Two, and two workgroups a compute unit, as
@@ -61,7 +61,7 @@ static __device__ __forceinline__ void load_to_shared(const void* base, uint32_t
 template <int GATED, int STAGES>
 __global__ void __launch_bounds__(256, STAGES == 2 ? 2 : 1)
 gemm_tile_kernel(const bf16* __restrict__ x, const bf16* __restrict__ w, bf16* __restrict__ out,
-                 float* __restrict__ partial, int M, int N, int K, int m_tiles, int k_per_split) {
+                 float* __restrict__ partial, int M, int N, int K, int m_tiles, int k_per_split, GateShape shape) {
     constexpr int kXRows = kTileRows, kWaves = 4;
     constexpr int kWBytes = kTileRows * kRowBytes, kXBytes = kXRows * kRowBytes;
     constexpr int kLoads = (kTileRows + kXRows) / 8 / kWaves;      // loads a wavefront and stage: 8 rows each
@@ -172,7 +172,7 @@ gemm_tile_kernel(const bf16* __restrict__ x, const bf16* __restrict__ w, bf16* _
 #pragma unroll
                 for (int v = 0; v < 4; ++v) {
                     const float gate = acc[a][b][v], up = acc[a + 2][b][v];
-                    r[v] = activate<(GATED > 0 ? GATED - 1 : 0)>(gate) * up;
+                    r[v] = gate_product<(GATED > 0 ? GATED - 1 : 0)>(gate, up, shape);
                 }
                 bf16* o = out + static_cast<size_t>(m) * N + n;
                 if (n + 3 < N && N % 4 == 0) {
@@ -219,19 +219,19 @@ gemm_tile_kernel(const bf16* __restrict__ x, const bf16* __restrict__ w, bf16* _
     }
 }
 
-// out[M, N] = x . w^T (gated 0, w [N, K]), or the gated product (gated = 1 + the activation's number;
-// w [2N, K], gate rows first).  splits > 1 (plain only): `out` is null and `partial` float32
+// out[M, N] = x . w^T (gated 0, w [N, K]), or the gated product (gated = 1 + the gate's number, with limit, slope and
+// shift for the clamped swish; w [2N, K], gate rows first).  splits > 1 (plain only): `out` is null and `partial` float32
 // [splits, M, N] takes the pieces' sums.  K must be a multiple of 64 * splits and the operands smaller
 // than 4 GiB.  Returns 0, a HIP error code, or -1 for sizes it does not take.
 WLLM_API int wllm_gemm_tile(const void* x, const void* w, void* out, float* partial, int M, int N, int K, int splits,
-                            int activation, hipStream_t stream) {
-    if (M < 1 || N < 1 || K < kStageKeys || splits < 1 || K % (kStageKeys * splits) != 0 || activation < 0 || activation > kActivations)
+                            int gated, float limit, float slope, float shift, hipStream_t stream) {
+    if (M < 1 || N < 1 || K < kStageKeys || splits < 1 || K % (kStageKeys * splits) != 0 || gated < 0 || gated > kGates)
         return -1;
-    if ((splits > 1) != (partial != nullptr) || (splits == 1 && out == nullptr) || (splits > 1 && activation != 0)) return -1;
-    const size_t w_rows = static_cast<size_t>(activation ? 2 : 1) * N;
+    if ((splits > 1) != (partial != nullptr) || (splits == 1 && out == nullptr) || (splits > 1 && gated != 0)) return -1;
+    const size_t w_rows = static_cast<size_t>(gated ? 2 : 1) * N;
     if (w_rows * K * 2 >= (size_t(1) << 32) || static_cast<size_t>(M) * K * 2 >= (size_t(1) << 32)) return -1;
     const int m_tiles = (M + kTileRows - 1) / kTileRows;
-    const int columns = activation ? kTileRows / 2 : kTileRows;
+    const int columns = gated ? kTileRows / 2 : kTileRows;
     const int n_tiles = (N + columns - 1) / columns;
     const long long blocks = static_cast<long long>((n_tiles + 7) / 8 * 8) * m_tiles;
     if (blocks > 0x7fffffffLL) return -1;
@@ -240,6 +240,7 @@ WLLM_API int wllm_gemm_tile(const void* x, const void* w, void* out, float* part
     const bf16* wp = static_cast<const bf16*>(w);
     bf16* op = static_cast<bf16*>(out);
     const int per = K / splits;
+    const GateShape shape{limit, slope, shift};
     constexpr int kStageBytes = 2 * kTileRows * kRowBytes;
 #define LAUNCH(GATED, STAGES)                                                                                      \
     do {                                                                                                            \
@@ -251,7 +252,7 @@ WLLM_API int wllm_gemm_tile(const void* x, const void* w, void* out, float* part
             roomy = true;                                                                                           \
         }                                                                                                           \
         gemm_tile_kernel<GATED, STAGES><<<grid, 256, STAGES * kStageBytes, stream>>>(xp, wp, op, partial, M, N, K,  \
-                                                                                     m_tiles, per);                 \
+                                                                                     m_tiles, per, shape);          \
     } while (0)
     // at most a workgroup a compute unit: nothing is lost by holding one, and it can have more on its way
     static int compute_units = 0;
@@ -265,8 +266,8 @@ WLLM_API int wllm_gemm_tile(const void* x, const void* w, void* out, float* part
 #define BY_STAGES(GATED)                \
     if (deep) LAUNCH(GATED, 4);         \
     else LAUNCH(GATED, 2)
-    if (activation == 0) { BY_STAGES(0); }
-    else { WLLM_BY_ACTIVATION(activation - 1, BY_STAGES(ACT + 1)) }
+    if (gated == 0) { BY_STAGES(0); }
+    else { WLLM_BY_GATE(gated - 1, BY_STAGES(GATE + 1)) }
 #undef BY_STAGES
 #undef LAUNCH
     return launch_status();

@@ -11,7 +11,7 @@ import torch
 
 from wllm_amd.kernels.attention_plan import AttentionPlan, build_work_items
 from wllm_amd.kernels import ops
-from wllm_amd.kernels.ops import ACTIVATIONS
+from wllm_amd.kernels.ops import gate_args
 from wllm_amd.kernels.library import load
 from wllm_amd.kernels.staging import pack_int32
 
@@ -36,9 +36,10 @@ _SIGNATURES = {
                       c_int, c_float, c_float, c_void_p],
     "wllm_rope_cache_write": [c_void_p, c_int, c_void_p, c_int, c_longlong, c_void_p, c_void_p, c_void_p, c_void_p,
                               c_void_p, c_longlong, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p],
-    "wllm_gemm_skinny_gated": [c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p],
+    "wllm_gemm_skinny_gated": [c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_int, c_float, c_float, c_float, c_int,
+                               c_int, c_void_p],
     "wllm_gemm_skinny_gated_norm": [c_void_p, c_void_p, c_int, c_void_p, c_float, c_float, c_void_p, c_int, c_void_p, c_int,
-                                    c_int, c_int, c_int, c_void_p],
+                                    c_int, c_int, c_int, c_float, c_float, c_float, c_void_p],
     "wllm_tile_weight": [c_void_p, c_void_p, c_int, c_int, c_void_p],
     "wllm_paged_attention_generic": [c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
                                      c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int,
@@ -56,7 +57,8 @@ _SIGNATURES = {
     "wllm_paged_attention_prefill": [c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_void_p, c_void_p, c_void_p,
                                      c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_float, c_int,
                                      c_int, c_float, c_int, c_void_p, c_void_p],
-    "wllm_gemm_tile": [c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p],
+    "wllm_gemm_tile": [c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_float, c_float, c_float,
+                       c_void_p],
     "wllm_split_sum": [c_void_p, c_void_p, c_int, c_longlong, c_int, c_void_p],
     "wllm_gemm_generic": [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_void_p],
     "wllm_tile_weight_f32": [c_void_p, c_void_p, c_int, c_int, c_void_p],
@@ -414,7 +416,7 @@ class HipBackend:
                 # sums the caller adds, or a kernel here in their order
                 n, splits = weight.shape[0], self.tile_splits(weight.shape[0], k, m)
                 stack = out if out.dim() == 3 else torch.empty((splits, m, n), dtype=torch.float32, device=x.device)
-                self._check(self.lib.wllm_gemm_tile(_ptr(x), _ptr(weight), None, _ptr(stack), m, n, k, splits, 0,
+                self._check(self.lib.wllm_gemm_tile(_ptr(x), _ptr(weight), None, _ptr(stack), m, n, k, splits, 0, 0.0, 0.0, 0.0,
                                                     self._stream()), "linear (tiles, partial sums)")
                 if out.dim() == 2:
                     self._check(self.lib.wllm_split_sum(_ptr(stack), _ptr(out), int(out.dtype == torch.bfloat16), m * n, splits,
@@ -483,7 +485,7 @@ class HipBackend:
         w, tiled = (tiles, 1) if tiles is not None else (weight, 0)
         if self.skinny_takes(x.dtype, m, k) and k % 64 == 0:
             self._check(self.lib.wllm_gemm_skinny_gated(
-                _ptr(x), _ptr(w), tiled, _ptr(out), m, out.shape[1], k, ACTIVATIONS[activation],
+                _ptr(x), _ptr(w), tiled, _ptr(out), m, out.shape[1], k, *gate_args(activation),
                 self.GATED_CHUNK[-(-m // 16)], out.stride(0) if m > 1 else out.shape[1], self._stream()),
                 "gated_linear (few rows, matrix cores)")
             return
@@ -491,8 +493,9 @@ class HipBackend:
         if (x.dtype == torch.bfloat16 and 64 < m <= self.TILE_GATED_MAX_ROWS and k % 64 == 0
                 and max(m, 2 * n) * k * 2 < 2 ** 32):
             # some hundred rows: the tiled product with the activation in its registers
-            self._check(self.lib.wllm_gemm_tile(_ptr(x), _ptr(weight), _ptr(out), None, m, n, k, 1,
-                                                1 + ACTIVATIONS[activation], self._stream()),
+            number, *shape = gate_args(activation)
+            self._check(self.lib.wllm_gemm_tile(_ptr(x), _ptr(weight), _ptr(out), None, m, n, k, 1, 1 + number, *shape,
+                                                self._stream()),
                         "gated_linear (tiles)")
             return
         # (the tile-major copy of a stacked float32 matrix is that of the one matrix it is; a bfloat16 one's
@@ -511,7 +514,7 @@ class HipBackend:
         w, tiled = (tiles, 1) if tiles is not None else (weight, 0)
         self._check(self.lib.wllm_gemm_skinny_gated_norm(
             _ptr(x.residual), _ptr(x.sumsq), x.sumsq.shape[1], _ptr(x.weight), x.eps, x.offset, _ptr(w), tiled,
-            _ptr(out), x.shape[0], out.shape[1], x.shape[1], ACTIVATIONS[activation], self._stream()),
+            _ptr(out), x.shape[0], out.shape[1], x.shape[1], *gate_args(activation), self._stream()),
             "gated_linear (norm on load)")
 
     ARGMAX_ROWS = 4096       # rows per launch; the scratch (64 words a row) is allocated once

@@ -14,6 +14,8 @@ emulation of each kernel's contract.
 from __future__ import annotations
 
 import contextlib
+import math
+from dataclasses import dataclass
 from typing import Optional
 
 import torch
@@ -587,10 +589,39 @@ def linear(x: torch.Tensor, weight: torch.Tensor, out: torch.Tensor, tiles: Opti
 ACTIVATIONS = {"gelu_tanh": 0, "silu": 1}
 
 
-def gated_activation(gate_up: torch.Tensor, out: torch.Tensor, activation: str) -> None:
-    """out = act(gate_up[:, :I]) * gate_up[:, I:], in float32, cast to T.  gate_up T [n, 2I]; out T [n, I],
-    possibly a band of columns of a wider tensor."""
-    _need(activation in ACTIVATIONS, lambda: f"activation {activation!r}: expected one of {sorted(ACTIVATIONS)}")
+@dataclass(frozen=True)
+class ClampedSwish:
+    """The step between a gated feed-forward's two products that holds both of its inputs under a limit:
+    g sigmoid(slope g) (u + shift) with g = min(gate, limit) and u = up held within -limit .. limit.  It stands
+    where the name of an activation stands in `gated_activation` and `gated_linear`."""
+    limit: float
+    slope: float = 1.0
+    shift: float = 0.0
+
+    def __post_init__(self):
+        for name in ("limit", "slope", "shift"):
+            if not math.isfinite(getattr(self, name)):
+                raise ValueError(f"{name} must be a finite number, got {getattr(self, name)}")
+        if not self.limit > 0:
+            raise ValueError(f"limit must be positive, got {self.limit}")
+
+
+def _known_gate(activation) -> None:
+    _need(isinstance(activation, ClampedSwish) or activation in ACTIVATIONS,
+          lambda: f"activation {activation!r}: expected one of {sorted(ACTIVATIONS)} or a ClampedSwish")
+
+
+def gate_args(activation) -> tuple:
+    """(number, limit, slope, shift) as the kernels of a gated feed-forward take them."""
+    if isinstance(activation, ClampedSwish):
+        return (len(ACTIVATIONS), activation.limit, activation.slope, activation.shift)
+    return (ACTIVATIONS[activation], 0.0, 0.0, 0.0)
+
+
+def gated_activation(gate_up: torch.Tensor, out: torch.Tensor, activation) -> None:
+    """out = act(gate_up[:, :I]) * gate_up[:, I:] (or a `ClampedSwish` of the two halves), in float32, cast to T.
+    gate_up T [n, 2I]; out T [n, I], possibly a band of columns of a wider tensor."""
+    _known_gate(activation)
     _dense(gate_up, "gate_up", _ACT)
     _need(gate_up.dim() == 2 and gate_up.shape[1] % 2 == 0, "gate_up: expected [n, 2*intermediate]")
     _band(out, "out", gate_up.dtype, gate_up.shape[0], gate_up.shape[1] // 2)
@@ -632,14 +663,15 @@ def gated_linear_writes_band(rows: int, dtype: torch.dtype, in_features: int) ->
     return bool(getattr(backend(), "gated_linear_writes_band", lambda *a: False)(rows, dtype, in_features))
 
 
-def gated_linear(x, weight: torch.Tensor, out: torch.Tensor, activation: str,
+def gated_linear(x, weight: torch.Tensor, out: torch.Tensor, activation,
                  scratch: Optional[torch.Tensor], tiles: Optional[torch.Tensor] = None) -> None:
-    """out = act(x @ Wg^T) * (x @ Wu^T) with weight = [Wg; Wu] stacked, T [2I, k]; x T [m, k];
+    """out = act(x @ Wg^T) * (x @ Wu^T) (or a `ClampedSwish` of the two products) with weight = [Wg; Wu] stacked,
+    T [2I, k]; x T [m, k];
     out T [m, I] (a band of a wider tensor where `gated_linear_writes_band`); scratch T [m, 2I] may be
     used for the unfused product.  `tiles` is
     `tile_weight(weight, halves=2)`.  x may be a `NormOnLoad` where `gated_linear_norm_takes` says so:
     the norm is then applied as the kernel reads the residual stream (scratch is not used)."""
-    _need(activation in ACTIVATIONS, lambda: f"activation {activation!r}: expected one of {sorted(ACTIVATIONS)}")
+    _known_gate(activation)
     if isinstance(x, NormOnLoad):
         _need(gated_linear_norm_takes(x.shape[0], x.dtype, x.shape[1]), "gated_linear: no kernel with the norm on load for these sizes")
         _dense(weight, "weight", x.dtype)
@@ -1245,9 +1277,9 @@ def _register_own() -> None:
                 launch=lambda fn, stream, ids, dst, src, source: fn(
                     p(ids), p(dst), p(src), p(source), dst.shape[0], ids.shape[0], source.shape[0], stream))
     register_op("gated_activation", entry_point="wllm_gated_activation",
-                argtypes=[c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_longlong, c_void_p],
+                argtypes=[c_void_p, c_void_p, c_int, c_int, c_float, c_float, c_float, c_int, c_int, c_longlong, c_void_p],
                 launch=lambda fn, stream, gate_up, out, activation: fn(
-                    p(gate_up), p(out), int(gate_up.dtype == torch.bfloat16), ACTIVATIONS[activation], gate_up.shape[0],
+                    p(gate_up), p(out), int(gate_up.dtype == torch.bfloat16), *gate_args(activation), gate_up.shape[0],
                     out.shape[1], out.stride(0) if out.shape[0] > 1 else out.shape[1], stream))
 
 

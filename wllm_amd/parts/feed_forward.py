@@ -1,5 +1,6 @@
 """Feed-forward parts.  "gated_mlp": down(act(gate(x)) * up(x)) without biases;
 with act = gelu_tanh it is the reference's GemmaMLP (src/wllm/models/gemma.py:54-62).
+"clamped_swish" holds the gate under a limit and the up projection between two, and raises the latter by a constant.
 Gate and up matrices are stacked at load so that one product makes both halves
 of the row the activation kernel reads."""
 from __future__ import annotations
@@ -16,8 +17,16 @@ from wllm_amd.weights.checkpoint import ExpectedTensor
 @register_feed_forward("gated_mlp")
 class GatedMLP:
     def __init__(self, spec: GatedMLPSpec):
-        if spec.activation not in ops.ACTIVATIONS:
-            raise ValueError(f"activation {spec.activation!r} is not implemented; known: {ops.ACTIVATIONS}")
+        if spec.activation == "clamped_swish":
+            if spec.gate_limit is None:
+                raise ValueError("a clamped swish needs gate_limit")
+            self.activation = ops.ClampedSwish(spec.gate_limit, spec.gate_slope, spec.up_shift)
+        elif spec.activation in ops.ACTIVATIONS:
+            if spec.gate_limit is not None or spec.gate_slope != 1.0 or spec.up_shift != 0.0:
+                raise ValueError(f"activation {spec.activation!r} takes no limit, slope or shift")
+            self.activation = spec.activation
+        else:
+            raise ValueError(f"activation {spec.activation!r} is not implemented; known: {ops.ACTIVATIONS} and clamped_swish")
         self.spec = spec
         self.w_gate_up = self.t_gate_up = None      # the matrix and its tile-major copy
         self.w_down = self.t_down = None
@@ -52,7 +61,7 @@ class GatedMLP:
         n = h.shape[0]
         if isinstance(h, ops.NormOnLoad):
             act = ctx.buffer("ffn_act", (n, s.intermediate_size), h.dtype)
-            ops.gated_linear(h, self.w_gate_up, act, s.activation, None, self.t_gate_up)
+            ops.gated_linear(h, self.w_gate_up, act, self.activation, None, self.t_gate_up)
         else:
             gate_up = ctx.buffer("gate_up", (n, 2 * s.intermediate_size), h.dtype)
             if (product_input is not None and ops.gated_linear_writes_band(n, h.dtype, s.hidden_size)
@@ -60,7 +69,7 @@ class GatedMLP:
                 act = product_input         # the kernel writes the band itself (its rows begin at multiples of 16 bytes)
             else:
                 act = ctx.buffer("ffn_act", (n, s.intermediate_size), h.dtype)
-            ops.gated_linear(h, self.w_gate_up, act, s.activation, gate_up, self.t_gate_up)
+            ops.gated_linear(h, self.w_gate_up, act, self.activation, gate_up, self.t_gate_up)
         if product_input is not None and act is not product_input:
             ops.copy_columns(act, product_input)
             act = product_input

@@ -133,7 +133,11 @@ class LatentAttentionSpec(MixerSpec):
     which the last r (not normed) are one more part of the key that all heads share; the r elements of the query heads
     and of that key part turn by the position, and the score is (q . k + q_r . k_r) * scale.  Cached: c and the turned
     key part.  `gate_weight` None: no gate.  `weights_in_float32`: the softmax weights are not rounded to the values' type
-    before they weigh the values."""
+    before they weigh the values.
+    `window` w: a query at position p sees the keys p-w+1..p.  `release_window`: the window by which the cache gives
+    pages back (the owner of a cache that layers with other windows read keeps what the widest of them needs; None
+    with `window` set: keep everything).  `owns_cache` False: the layer has no W_dkv (nor its norm); its W_uk and W_uv
+    expand the vectors that the schedule entry its run names keeps in its cache, of the same kv_rank."""
     kind: str = "latent_attention"
     hidden_size: int = 0
     num_heads: int = 0
@@ -157,6 +161,9 @@ class LatentAttentionSpec(MixerSpec):
     rope_dim: int = 0
     position: PositionSpec = field(default_factory=lambda: PositionSpec(kind="none"))
     weights_in_float32: bool = False
+    window: Optional[int] = None
+    release_window: Optional[int] = None
+    owns_cache: bool = True
 
 
 @dataclass(frozen=True)
@@ -268,7 +275,8 @@ class FeedForwardSpec:
 @dataclass(frozen=True)
 class GatedMLPSpec(FeedForwardSpec):
     """down(act(gate(x)) * up(x)) without biases; `activation` names the
-    nonlinearity ("gelu_tanh")."""
+    nonlinearity ("gelu_tanh", "silu").  "clamped_swish": down(g sigmoid(gate_slope g) (u + up_shift)) with
+    g = min(gate(x), gate_limit) and u = up(x) held within -gate_limit .. gate_limit."""
     kind: str = "gated_mlp"
     hidden_size: int = 0
     intermediate_size: int = 0
@@ -276,6 +284,9 @@ class GatedMLPSpec(FeedForwardSpec):
     gate_weight: str = ""
     up_weight: str = ""
     down_weight: str = ""
+    gate_limit: Optional[float] = None
+    gate_slope: float = 1.0
+    up_shift: float = 0.0
 
 
 @dataclass(frozen=True)
