@@ -121,6 +121,30 @@ def test_the_limit_with_the_norm_on_load():
     close(out, want, torch.bfloat16, scale=2.0)
 
 
+@pytest.mark.parametrize("n,heads,outs,keys", [(1, 3, 96, 32), (16, 5, 40, 24), (17, 2, 256, 128), (33, 3, 30, 8), (64, 16, 256, 128),
+                                               (300, 4, 128, 256), (1100, 16, 250, 40), (1030, 16, 256, 64), (129, 7, 18, 56)])
+def test_products_head_by_head_on_the_matrix_cores(n, heads, outs, keys):
+    """bfloat16 bands whose rows begin at multiples of 16 bytes; every row has the bits it has alone or among any others,
+    and nothing beside the band is written."""
+    g = torch.Generator().manual_seed(n + keys)
+    wide = torch.randn(n, heads * keys + 16, generator=g).to(torch.bfloat16)
+    wide[:, :8], wide[:, heads * keys + 8:] = float("nan"), float("nan")
+    w = (torch.randn(heads, outs, keys, generator=g) * keys ** -0.5).to(torch.bfloat16)
+    x, wd = wide.to(DEV)[:, 8:heads * keys + 8], w.to(DEV)
+
+    def made(lo, hi):
+        y = torch.full((hi - lo, heads * outs + 8), 3.0, dtype=torch.bfloat16, device=DEV)
+        ops.head_linear(x[lo:hi], wd, y[:, :heads * outs])
+        assert (y[:, heads * outs:] == 3.0).all()
+        return y[:, :heads * outs]
+
+    got = made(0, n)
+    want = torch.stack([wide[:, 8 + h * keys:8 + (h + 1) * keys].double() @ w[h].double().T for h in range(heads)], 1)
+    close(got, want.reshape(n, -1), torch.bfloat16)
+    for lo, hi in ((0, 1), (n // 2, min(n, n // 2 + 5)), (max(0, n - 20), n), (0, min(n, 50))):
+        assert torch.equal(made(lo, hi), got[lo:hi])
+
+
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("hidden,stack", [(64, 0), (300, 3), (2048, 0), (48, 2), (3072, 4)])
 def test_a_norm_behind_a_sublayer_and_the_stream_as_the_next_one_reads_it(dtype, hidden, stack):

@@ -265,7 +265,8 @@ WLLM_API int wllm_gated_lookup(const void* gate, const int* ids, const void* tab
 
 // ---- a product head by head: y[r, h * O + o] = sum_k x[r, h * K + k] * w[h, o, k].  x and y are
 // bands of wider tensors (row strides); w is [heads, O, K].  float32 sums in ascending order of k,
-// so a row's result does not depend on the rows beside it.  A workgroup makes 32 rows by 64 outputs
+// so a row's result does not depend on the rows beside it.  bfloat16 goes to the matrix cores (further
+// below) where its rows are aligned; the kernels on the vector units here take everything.  A workgroup makes 32 rows by 64 outputs
 // of one head, a thread 2 by 4 of them, from chunks of 32 keys staged in shared memory. ----
 constexpr int kHlRows = 32, kHlOuts = 64, kHlKeys = 32;
 
@@ -391,10 +392,109 @@ head_linear_few_kernel(const T* __restrict__ x, long long x_stride, const T* __r
     }
 }
 
+// The same for bfloat16 on the matrix cores (keys in multiples of 8, rows that begin at multiples of 16 bytes).  A
+// wavefront makes 16 MT rows by 16 NT outputs of one head with v_mfma_f32_16x16x32_bf16: w is the A operand (lane
+// (i, g) holds keys 8 g .. + 7 of output i), x the B operand (the same keys of row i), both straight from memory, 16
+// bytes a lane; the result lands as four consecutive outputs of row i a lane.  The keys go by in steps of 32 from the
+// first, the last step filled with zeros, whatever MT and NT are, so a row has the same bits in any batch.
+typedef __bf16 hl_bf16x8 __attribute__((ext_vector_type(8)));
+typedef float hl_float4 __attribute__((ext_vector_type(4)));
+union HlFrag {
+    uint4 u;
+    hl_bf16x8 v;
+};
+
+template <int MT, int NT>
+__global__ void __launch_bounds__(256)
+head_linear_mfma_kernel(const bf16* __restrict__ x, long long x_stride, const bf16* __restrict__ w, bf16* __restrict__ y,
+                        long long y_stride, int rows, int outs, int keys, int out_tiles, int tiles, int whole_stores) {
+    const int lane = threadIdx.x % kWave, wave = threadIdx.x / kWave;
+    const int i = lane % 16, g = lane / 16;
+    const int h = blockIdx.y, tile = blockIdx.x * (blockDim.x / kWave) + wave;
+    if (tile >= tiles) return;
+    const int o0 = (tile % out_tiles) * 16 * NT, r0 = (tile / out_tiles) * 16 * MT;
+    // rows and outputs beyond the last read the last one: what comes of them is not written
+    const bf16* wp[NT];
+    const bf16* xp[MT];
+#pragma unroll
+    for (int a = 0; a < NT; ++a)
+        wp[a] = w + (static_cast<size_t>(h) * outs + min(o0 + 16 * a + i, outs - 1)) * keys + 8 * g;
+#pragma unroll
+    for (int b = 0; b < MT; ++b)
+        xp[b] = x + static_cast<size_t>(min(r0 + 16 * b + i, rows - 1)) * x_stride + static_cast<size_t>(h) * keys + 8 * g;
+    hl_float4 acc[NT][MT];
+#pragma unroll
+    for (int a = 0; a < NT; ++a)
+#pragma unroll
+        for (int b = 0; b < MT; ++b) acc[a][b] = hl_float4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+    for (int k = 0; k < keys; k += 32) {
+        const bool in = k + 8 * g < keys;
+        HlFrag fw[NT], fx[MT];
+#pragma unroll
+        for (int a = 0; a < NT; ++a) fw[a].u = in ? *reinterpret_cast<const uint4*>(wp[a] + k) : make_uint4(0, 0, 0, 0);
+#pragma unroll
+        for (int b = 0; b < MT; ++b) fx[b].u = in ? *reinterpret_cast<const uint4*>(xp[b] + k) : make_uint4(0, 0, 0, 0);
+#pragma unroll
+        for (int a = 0; a < NT; ++a)
+#pragma unroll
+            for (int b = 0; b < MT; ++b)
+                acc[a][b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(fw[a].v, fx[b].v, acc[a][b], 0, 0, 0);
+    }
+#pragma unroll
+    for (int b = 0; b < MT; ++b) {
+        const int r = r0 + 16 * b + i;
+        if (r >= rows) continue;
+        bf16* yr = y + static_cast<size_t>(r) * y_stride + static_cast<size_t>(h) * outs;
+#pragma unroll
+        for (int a = 0; a < NT; ++a) {
+            const int o = o0 + 16 * a + 4 * g;
+            if (whole_stores && o + 3 < outs) {
+                uint2 p;
+                p.x = pack2_bf16(acc[a][b][0], acc[a][b][1]);
+                p.y = pack2_bf16(acc[a][b][2], acc[a][b][3]);
+                *reinterpret_cast<uint2*>(yr + o) = p;
+            } else {
+#pragma unroll
+                for (int v = 0; v < 4; ++v)
+                    if (o + v < outs) yr[o + v] = from_float<bf16>(acc[a][b][v]);
+            }
+        }
+    }
+}
+
+static int head_linear_mfma(const bf16* x, long long x_stride, const bf16* w, bf16* y, long long y_stride, int rows, int heads,
+                            int outs, int keys, hipStream_t stream) {
+    const int whole = outs % 4 == 0 && y_stride % 4 == 0 && reinterpret_cast<uintptr_t>(y) % 8 == 0;
+    const int mt = rows <= 16 ? 1 : rows <= 32 ? 2 : 4;
+    // four tiles of outputs a wavefront where about a thousand wavefronts remain
+    const long long row_tiles = (rows + 16 * mt - 1) / (16 * mt);
+    const int nt = mt == 4 && row_tiles * ((outs + 63) / 64) * heads >= 1024 ? 4 : 1;
+    const int out_tiles = (outs + 16 * nt - 1) / (16 * nt);
+    const long long tiles = row_tiles * out_tiles;
+    const int waves = tiles * heads >= 1024 ? 4 : 1;
+    if (tiles > 0x7fffffffLL) return -1;
+    const dim3 grid(static_cast<unsigned>((tiles + waves - 1) / waves), heads);
+#define LAUNCH(MT, NT)                                                                                                 \
+    head_linear_mfma_kernel<MT, NT><<<grid, waves * kWave, 0, stream>>>(x, x_stride, w, y, y_stride, rows, outs, keys, \
+                                                                        out_tiles, static_cast<int>(tiles), whole)
+    if (mt == 1) LAUNCH(1, 1);
+    else if (mt == 2) LAUNCH(2, 1);
+    else if (nt == 1) LAUNCH(4, 1);
+    else LAUNCH(4, 4);
+#undef LAUNCH
+    return launch_status();
+}
+
 WLLM_API int wllm_head_linear(const void* x, long long x_stride, const void* w, void* y, long long y_stride, int is_bf16,
                               int rows, int heads, int outs, int keys, hipStream_t stream) {
     if (rows <= 0) return 0;
     if (heads <= 0 || outs <= 0 || keys <= 0 || heads > 65535) return -1;
+    // (the last row's band may end where the tensor does: whole pieces of 8 keys stay inside it)
+    if (is_bf16 && keys % 8 == 0 && x_stride % 8 == 0 && reinterpret_cast<uintptr_t>(x) % 16 == 0 &&
+        reinterpret_cast<uintptr_t>(w) % 16 == 0)
+        return head_linear_mfma(static_cast<const bf16*>(x), x_stride, static_cast<const bf16*>(w), static_cast<bf16*>(y), y_stride,
+                                rows, heads, outs, keys, stream);
     const dim3 grid((rows + kHlRows - 1) / kHlRows, heads, (outs + kHlOuts - 1) / kHlOuts);
     if (grid.z > 65535) return -1;
     const size_t smem = sizeof(float) * (static_cast<size_t>(rows) * keys + 4 * static_cast<size_t>(rows) * kHlOuts);

@@ -849,7 +849,7 @@ def gated_lookup(gate: torch.Tensor, ids: torch.Tensor, table: torch.Tensor, col
 
 def head_linear(x: torch.Tensor, w: torch.Tensor, y: torch.Tensor) -> None:
     """A product head by head: y[r, h*O + o] = sum_k x[r, h*K + k] * w[h, o, k], float32 sums in ascending
-    order of k.  x T [n, heads*K] and y T [n, heads*O] may be bands of wider tensors; w T [heads, O, K]."""
+    order of k (on the matrix cores, where they take the sizes, 32 at a time).  x T [n, heads*K] and y T [n, heads*O] may be bands of wider tensors; w T [heads, O, K]."""
     _dense(w, "w", _ACT)
     _need(w.dim() == 3, "w: expected [heads, out, in]")
     heads, o, k = w.shape
