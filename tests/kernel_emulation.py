@@ -181,7 +181,8 @@ class EmulatedKernels:
         return None
 
     def head_prepare(self, rows, bias, positions, inv_freq, slots, cache, num_heads, num_kv_heads, head_dim, page_size,
-                     interleaved, norm_eps, values_are_keys, parts, norm_dim=None, head_norm=None, rot_scale=1.0):
+                     interleaved, norm_eps, values_are_keys, parts, norm_dim=None, head_norm=None, rot_scale=1.0,
+                     q_temperature=None):
         self._count("head_prepare")
         n, width = rows.shape
         if parts is not None:
@@ -216,6 +217,10 @@ class EmulatedKernels:
                 heads[..., half:2 * half] = x2 * cos + x1 * sin
         if norm_eps is not None:
             heads = heads * torch.rsqrt(heads.pow(2).sum(-1, keepdim=True) / (norm_dim or head_dim) + norm_eps)
+        if q_temperature is not None:
+            coef, every = q_temperature
+            turns = torch.div(positions + 1, every, rounding_mode="floor").to(self.acc)
+            heads[:, :num_heads] *= (1.0 + coef * torch.log(turns + 1.0))[:, None, None]
         v[:, :r * head_dim] = heads.reshape(n, -1)
         rows.copy_(v.to(rows.dtype))
         if cache is not None:
@@ -244,7 +249,16 @@ class EmulatedKernels:
             v = v - v.mean(-1, keepdim=True)
         return v * torch.rsqrt(v.pow(2).mean(-1, keepdim=True) + recipe.eps) * (recipe.offset + recipe.weight.to(self.acc))
 
-    def norm_add(self, x, delta, delta_norm, out, out_norm, rows, conv=None):
+    def _stack(self, t):
+        if t.dim() == 2:
+            return t
+        total = t[0]
+        for p in range(1, t.shape[0]):
+            total = total + t[p]
+        return total
+
+    def norm_add(self, x, delta, delta_norm, out, out_norm, rows, conv=None, x_scale=1.0, sum_norm=None, extra=None,
+                 extra_scale=None):
         self._count("norm_add")
         idx = rows.long() if rows is not None else slice(None)
         v = x[idx].to(self.acc)
@@ -254,7 +268,11 @@ class EmulatedKernels:
                 for p in range(1, delta.shape[0]):
                     total = total + delta[p]
                 delta = total
-            v = (v + self._normed(delta[idx].to(self.acc), delta_norm)).to(x.dtype)
+            d = delta[idx].to(self.acc)
+            if extra is not None:
+                e = self._stack(extra)[idx].to(self.acc)
+                d = d + (e if extra_scale is None else e * extra_scale[idx].to(self.acc)[:, None])
+            v = self._normed(x_scale * v + self._normed(d, delta_norm), sum_norm).to(x.dtype)
             if rows is None:
                 x.copy_(v)
             v = v.to(self.acc)
@@ -463,23 +481,79 @@ class EmulatedKernels:
             v = v * (torch.sigmoid(z) if activation == "sigmoid" else z * torch.sigmoid(z))
         out.copy_((v * scale).to(out.dtype))
 
+    # ---- a delta rule with a decay a key channel ----------------------------------------------------
+    def delta_inputs(self, xqkv, z, b, conv_weight, rate, dt_bias, state, carried_offset, token_segment, seg_q_start,
+                     seg_q_len, state_slots, qk, kq, v, f, beta, heads, groups, head_dim, value_dim, q_scale, unit_eps,
+                     single_tokens):
+        self._count("delta_inputs")
+        assert not single_tokens or all(int(n) == 1 for n in seg_q_len)
+        acc, n = self.acc, xqkv.shape[0]
+        taps, c = conv_weight.shape
+        out = torch.zeros(n, c, dtype=acc)
+        for s in range(seg_q_start.shape[0]):
+            q0, ql, slot = int(seg_q_start[s]), int(seg_q_len[s]), int(state_slots[s])
+            if ql == 0:
+                continue
+            carried = state[slot, carried_offset:carried_offset + (taps - 1) * c].view(taps - 1, c)
+            seq = torch.cat([carried.to(acc), xqkv[q0:q0 + ql].to(acc)], dim=0)
+            for k in range(taps):
+                out[q0:q0 + ql] += seq[k:k + ql] * conv_weight[k].to(acc)
+            if taps > 1:
+                carried.copy_(seq[ql:].float())
+        out = out * torch.sigmoid(out)
+        gd, dp = groups * head_dim, qk.shape[2] // groups
+        unit = lambda t: t / torch.sqrt((t * t).sum(-1, keepdim=True) + unit_eps)
+        q = unit(out[:, :gd].view(n, groups, head_dim)) * q_scale
+        k = unit(out[:, gd:2 * gd].view(n, groups, head_dim))
+        qk.zero_()
+        qk[0].view(n, groups, dp)[..., :head_dim] = q.float()
+        qk[1].view(n, groups, dp)[..., :head_dim] = k.float()
+        kq.copy_((q * k).sum(-1).float())
+        v.copy_(out[:, 2 * gd:].to(v.dtype))
+        dt = torch.nn.functional.softplus(z.to(acc) + dt_bias.to(acc), threshold=1e9).view(n, heads, head_dim)
+        f.zero_()
+        f.view(n, heads, dp)[..., :head_dim] = torch.exp(-rate.to(acc)[:, None] * dt).float()
+        beta.copy_(torch.sigmoid(b.to(acc)).float())
+
+    def delta_scan(self, qk, kq, f, beta, v, state, seg_q_start, seg_q_len, state_slots, y, heads, groups, head_dim, value_dim):
+        self._count("delta_scan")
+        acc = self.acc
+        dp, per = f.shape[1] // heads, heads // groups
+        size = heads * value_dim * dp
+        for s in range(seg_q_start.shape[0]):
+            q0, ql, slot = int(seg_q_start[s]), int(seg_q_len[s]), int(state_slots[s])
+            S = state[slot, :size].to(acc).view(heads, value_dim, dp).clone()
+            for t in range(q0, q0 + ql):
+                q, k = (qk[i, t].to(acc).view(groups, dp).repeat_interleave(per, dim=0) for i in range(2))
+                S = S * f[t].to(acc).view(heads, 1, dp)
+                u = beta[t].to(acc)[:, None] * (v[t].to(acc).view(heads, value_dim) - (S * k[:, None]).sum(-1))
+                S = S + u[:, :, None] * k[:, None]
+                y[t] = (S * q[:, None]).sum(-1).reshape(-1).float()
+            if ql:
+                state[slot, :size] = S.reshape(-1).float()
+
     # ---- a mixture of experts ---------------------------------------------------------------------
-    def moe_route(self, x, router, ids, weights, groups, keep, eps, scoring="softmax", normalize=True):
+    def moe_route(self, x, router, ids, weights, groups, keep, eps, scoring="softmax", normalize=True, correction=None,
+                  group_best=1, gates=None):
         self._count("moe_route")
-        n, experts, top = x.shape[0], router.shape[0], ids.shape[1]
+        n, experts, top = x.shape[0], router.shape[0] - (1 if gates is not None else 0), ids.shape[1]
         z = x.to(self.acc) @ router.to(self.acc).T
+        if gates is not None:
+            gates.copy_(torch.sigmoid(z[:, experts]).float())
+            z = z[:, :experts]
         s = torch.sigmoid(z) if scoring == "sigmoid" else torch.softmax(z, dim=-1)
+        c = s if correction is None else s + correction.to(self.acc)
         allowed = torch.ones(n, experts, dtype=torch.bool)
         if keep < groups:
             per = experts // groups
-            best = s.view(n, groups, per).max(-1).values
+            best = c.view(n, groups, per).topk(min(group_best, per), dim=-1).values.sum(-1)
             kept = torch.zeros(n, groups, dtype=torch.bool)
             for r in range(n):
                 order = sorted(range(groups), key=lambda g: (-float(best[r, g]), g))
                 kept[r, order[:keep]] = True
             allowed = kept[:, :, None].expand(n, groups, per).reshape(n, experts)
         for r in range(n):
-            order = sorted([e for e in range(experts) if allowed[r, e]], key=lambda e: (-float(s[r, e]), e))[:top]
+            order = sorted([e for e in range(experts) if allowed[r, e]], key=lambda e: (-float(c[r, e]), e))[:top]
             chosen = s[r, order]
             ids[r] = torch.tensor(order, dtype=torch.int32)
             weights[r] = (chosen / (chosen.sum() + eps) if normalize else chosen).float()
@@ -635,6 +709,22 @@ class EmulatedKernels:
         else:
             raise ValueError(activation)
         out.copy_((a * u).to(out.dtype))
+
+    def activation(self, x, out, name):
+        self._count("activation")
+        z = x.to(self.acc)
+        if name == "gelu_tanh":
+            a = 0.5 * z * (1.0 + torch.tanh(math.sqrt(2.0 / math.pi) * (z + 0.044715 * z.pow(3))))
+        else:
+            a = z * torch.sigmoid(z) if name == "silu" else torch.clamp(z, min=0.0).pow(2)
+        out.copy_(a.to(out.dtype))
+
+    def activated_linear(self, x, weight, out, name, tiles=None, paired_tiles=None):
+        self._count("activated_linear")
+        self._same_numbers(weight, tiles, 1)
+        self._same_numbers(weight, paired_tiles, 2)
+        self.activation(x.to(self.acc) @ weight.to(self.acc).T, out, name)
+        self.calls["activation"] -= 1
 
     def argmax_rows(self, logits, out):
         self._count("argmax_rows")

@@ -168,10 +168,27 @@ __device__ __forceinline__ float activate(float z) {
 // others do not read it).
 constexpr int kGateClampedSwish = kActivations;
 constexpr int kGates = kActivations + 1;
+// Behind these, for the product kernels alone, a "gate" that is none: the two halves of the product are two halves of
+// one ungated feed-forward's columns, and each takes the squared relu by itself (`kPairedGates` counts it).
+constexpr int kGatePairSquaredRelu = kGates;
+constexpr int kPairedGates = kGates + 1;
+
+// The activations of a feed-forward without a gate, by the number the host passes: those above, and the squared relu.
+constexpr int kActSquaredRelu = kActivations;
+constexpr int kSingleActivations = kActivations + 1;
 
 struct GateShape {
     float limit, slope, shift;
 };
+
+// (a comparison, not fmaxf: what is not a number stays visible)
+__device__ __forceinline__ float squared_relu(float z) { return z < 0.f ? 0.f : z * z; }
+
+template <int ACT>
+__device__ __forceinline__ float activate_single(float z) {
+    if (ACT == kActSquaredRelu) return squared_relu(z);
+    return activate<(ACT < kActivations ? ACT : 0)>(z);
+}
 
 template <int GATE>
 __device__ __forceinline__ float gate_product(float gate, float up, GateShape shape) {
@@ -189,6 +206,15 @@ __device__ __forceinline__ float gate_product(float gate, float up, GateShape sh
         case kActGeluTanh: { constexpr int GATE = kActGeluTanh; statement; } break;          \
         case kActSilu: { constexpr int GATE = kActSilu; statement; } break;                  \
         default: { constexpr int GATE = kGateClampedSwish; statement; } break;               \
+    }
+
+// The same with the paired squared relu among the gates.
+#define WLLM_BY_PAIRED_GATE(gate, statement)                                                 \
+    switch (gate) {                                                                          \
+        case kActGeluTanh: { constexpr int GATE = kActGeluTanh; statement; } break;          \
+        case kActSilu: { constexpr int GATE = kActSilu; statement; } break;                  \
+        case kGateClampedSwish: { constexpr int GATE = kGateClampedSwish; statement; } break; \
+        default: { constexpr int GATE = kGatePairSquaredRelu; statement; } break;            \
     }
 
 // Runs `statement` with the compile-time constant ACT set to the activation's number.

@@ -1,0 +1,323 @@
+// A gated delta rule whose decay is a number a head and key channel, on a flat batch of segments.  A segment is the
+// next tokens of one request; what a request carries from step to step lies in one float32 row of `state` per request
+// (row state_slots[segment]):
+//   [heads, P, DP] the memory, a column of P after the other (its D key channels, padded with zeros to DP = a multiple of
+//   four), then [taps - 1, channels] the last inputs of the short convolutions (the oldest first).
+// A fresh request's row is all zeros: the memory and what lies before the start.  Per head and token
+//   S = diag(g) S;   u = beta (v - S^T k);   S = S + k u^T;   o = S^T q
+// with k and q unit vectors (q times a factor).  Everything behind the projections and the convolutions is float32: unit
+// norms, step sizes, decays, beta, the memory and every sum.
+#include "common.h"
+#include "short_conv.h"
+
+__device__ __forceinline__ float delta_softplus(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
+
+// ---- what the recurrence reads, from a token's projections:
+//   q, k, v   silu(short convolution) of their bands of the row (`xqkv`: groups * D, groups * D, heads * P columns, in the
+//             weights' order); q and k then unit vectors a head, x / sqrt(sum(x^2) + unit_eps), q times q_scale
+//   kq        k . q of every group
+//   f         exp(-rate * softplus(z + dt_bias)) a head and channel, rate = exp(A_log) of the head
+//   beta      sigmoid of its projection
+// qk float32 [2, tokens, groups * DP] (channels beyond D are zeros), kq float32 [tokens, groups], v T [tokens, heads * P],
+// f float32 [tokens, heads * DP], beta float32 [tokens, heads].
+// The grid is (token, piece): a wavefront takes one group's q and k, or 256 of the other results.  CARRY (a step of single
+// tokens): the threads that read a request's carried rows move them up by one; else `conv_carry_kernel` does that. ----
+constexpr int kDeltaWaves = 4;
+constexpr int kDeltaPer = 4;                    // elements a lane: heads of up to 256 channels
+
+struct DeltaInputs {
+    const float* conv_w;                        // [taps, channels], a row a tap
+    float* state;
+    long long state_stride, carried_offset;
+    const int* token_segment;
+    const int* seg_q_start;
+    const int* state_slots;
+    const float* rate;
+    const float* dt_bias;
+    float* qk;
+    float* kq;
+    float* f;
+    float* beta;
+    float q_scale, unit_eps;
+    int tokens, heads, groups, d, dp, p_dim, taps;
+};
+
+template <typename T, bool CARRY>
+__global__ void __launch_bounds__(kWave * kDeltaWaves)
+delta_inputs_kernel(const T* __restrict__ xqkv, long long x_stride, const T* __restrict__ z, long long z_stride,
+                    const T* __restrict__ b, long long b_stride, T* __restrict__ v, DeltaInputs a) {
+    const int token = blockIdx.x;
+    const int lane = threadIdx.x % kWave, wave = threadIdx.x / kWave;
+    const int seg = a.token_segment[token];
+    const int local = token - a.seg_q_start[seg];
+    const int channels = 2 * a.groups * a.d + a.heads * a.p_dim;
+    float* carried = a.state + static_cast<size_t>(a.state_slots[seg]) * a.state_stride + a.carried_offset;
+    const T* xt = xqkv + static_cast<size_t>(token) * x_stride;
+    auto convolved = [&](int c) -> float {
+        return short_conv<T, CARRY>(xt, x_stride, local, carried, a.conv_w, channels, a.taps, c);
+    };
+    int unit = blockIdx.y * kDeltaWaves + wave;
+    if (unit < a.groups) {
+        float q[kDeltaPer], k[kDeltaPer], qq = 0.f, kk = 0.f;
+#pragma unroll
+        for (int j = 0; j < kDeltaPer; ++j) {
+            const int i = lane + kWave * j;
+            q[j] = k[j] = 0.f;
+            if (i < a.d) {
+                q[j] = convolved(unit * a.d + i);
+                k[j] = convolved((a.groups + unit) * a.d + i);
+            }
+            qq = fmaf(q[j], q[j], qq);
+            kk = fmaf(k[j], k[j], kk);
+        }
+        const float q_inv = a.q_scale / sqrtf(wave_sum(qq) + a.unit_eps), k_inv = 1.f / sqrtf(wave_sum(kk) + a.unit_eps);
+        const size_t width = static_cast<size_t>(a.groups) * a.dp;
+        float* q_out = a.qk + static_cast<size_t>(token) * width + static_cast<size_t>(unit) * a.dp;
+        float* k_out = q_out + static_cast<size_t>(a.tokens) * width;
+        float dot = 0.f;
+#pragma unroll
+        for (int j = 0; j < kDeltaPer; ++j) {
+            const int i = lane + kWave * j;
+            q[j] *= q_inv;
+            k[j] *= k_inv;
+            dot = fmaf(q[j], k[j], dot);
+            if (i < a.dp) {
+                q_out[i] = q[j];
+                k_out[i] = k[j];
+            }
+        }
+        dot = wave_sum(dot);
+        if (lane == 0) a.kq[static_cast<size_t>(token) * a.groups + unit] = dot;
+        return;
+    }
+    unit -= a.groups;
+    const int v_width = a.heads * a.p_dim, f_width = a.heads * a.dp;
+#pragma unroll
+    for (int j = 0; j < kDeltaPer; ++j) {
+        int e = unit * kWave * kDeltaPer + kWave * j + lane;
+        if (e < v_width) {
+            v[static_cast<size_t>(token) * v_width + e] = from_float<T>(convolved(2 * a.groups * a.d + e));
+            continue;
+        }
+        e -= v_width;
+        if (e < f_width) {
+            const int h = e / a.dp, i = e - h * a.dp;
+            float f = 0.f;
+            if (i < a.d) {
+                const int c = h * a.d + i;
+                f = expf(-a.rate[h] * delta_softplus(to_float(z[static_cast<size_t>(token) * z_stride + c]) + a.dt_bias[c]));
+            }
+            a.f[static_cast<size_t>(token) * f_width + e] = f;
+            continue;
+        }
+        e -= f_width;
+        if (e < a.heads)
+            a.beta[static_cast<size_t>(token) * a.heads + e] = 1.f / (1.f + expf(-to_float(b[static_cast<size_t>(token) * b_stride + e])));
+    }
+}
+
+WLLM_API int wllm_delta_inputs(const void* xqkv, long long x_stride, const void* z, long long z_stride, const void* b,
+                               long long b_stride, const float* conv_w, const float* rate, const float* dt_bias, float* state,
+                               long long state_stride, long long carried_offset, const int* token_segment, const int* seg_q_start,
+                               const int* seg_q_len, const int* state_slots, float* qk, float* kq, void* v, float* f, float* beta,
+                               float q_scale, float unit_eps, int is_bf16, int tokens, int segments, int heads, int groups, int d,
+                               int p_dim, int taps, int single_tokens, hipStream_t stream) {
+    if (tokens <= 0 || segments <= 0) return 0;
+    if (heads <= 0 || groups <= 0 || heads % groups || d <= 0 || d > kWave * kDeltaPer || p_dim <= 0 || taps < 1 || taps > 64) return -1;
+    if (single_tokens && tokens != segments) return -1;
+    const int dp = (d + 3) / 4 * 4;
+    const long long rest = static_cast<long long>(heads) * (p_dim + dp + 1);
+    const long long units = groups + (rest + kWave * kDeltaPer - 1) / (kWave * kDeltaPer);
+    const long long pieces = (units + kDeltaWaves - 1) / kDeltaWaves;
+    if (pieces > 65535) return -1;
+    const DeltaInputs a{conv_w, state, state_stride, carried_offset, token_segment, seg_q_start, state_slots, rate, dt_bias, qk, kq, f,
+                        beta, q_scale, unit_eps, tokens, heads, groups, d, dp, p_dim, taps};
+    const dim3 grid(tokens, static_cast<unsigned>(pieces));
+#define LAUNCH(T, CARRY)                                                                                                \
+    delta_inputs_kernel<T, CARRY><<<grid, kWave * kDeltaWaves, 0, stream>>>(                                            \
+        static_cast<const T*>(xqkv), x_stride, static_cast<const T*>(z), z_stride, static_cast<const T*>(b), b_stride,  \
+        static_cast<T*>(v), a)
+    if (is_bf16) { if (single_tokens) LAUNCH(bf16, true); else LAUNCH(bf16, false); }
+    else { if (single_tokens) LAUNCH(float, true); else LAUNCH(float, false); }
+#undef LAUNCH
+    if (const int err = launch_status()) return err;
+    if (taps == 1 || single_tokens) return 0;
+    const int channels = 2 * groups * d + heads * p_dim;
+    const dim3 carry_grid(segments, (channels + 255) / 256 < 64 ? (channels + 255) / 256 : 64);
+    if (is_bf16)
+        conv_carry_kernel<bf16><<<carry_grid, 256, 0, stream>>>(static_cast<const bf16*>(xqkv), x_stride, state, state_stride,
+                                                                carried_offset, seg_q_start, seg_q_len, state_slots, channels, taps);
+    else
+        conv_carry_kernel<float><<<carry_grid, 256, 0, stream>>>(static_cast<const float*>(xqkv), x_stride, state, state_stride,
+                                                                 carried_offset, seg_q_start, seg_q_len, state_slots, channels, taps);
+    return launch_status();
+}
+
+// ---- the recurrence.  The columns of a head's memory do not depend on each other, and a column's new write needs the
+// sum over all its channels first: a column lies within 16 lanes, lane s of them holding the channels 4s .. 4s + 3 (and
+// those 64, 128, 192 further on) in registers, and both sums of a token (S^T k and S^T q of the decayed memory) go
+// through the 16 lanes by the vector unit's own permutations; the read-out behind the write is then S^T q + u (k . q).
+// A wavefront is four columns, a workgroup's four wavefronts sixteen; nothing passes between them but the tokens' k, q
+// and f, which go 16 tokens at a time through shared memory, the next 16 fetched into registers while these are
+// walked.  A token's results are the same operations in the same order however the tokens are cut into steps. ----
+constexpr int kScanTokens = 16;
+constexpr int kScanWaves = 4;
+constexpr int kScanLanes = 16;                               // lanes a column
+constexpr int kScanCols = kWave / kScanLanes * kScanWaves;   // columns a workgroup
+constexpr int kScanThreads = kWave * kScanWaves;
+
+__device__ __forceinline__ float row_sum(float v) {          // over the 16 lanes of a row, in every lane
+    v += row_permuted<0x128>(v);
+    v += row_permuted<0x124>(v);
+    v += row_permuted<0x4E>(v);
+    v += row_permuted<0xB1>(v);
+    return v;
+}
+
+template <typename T, int R>        // R: groups of four channels a lane (heads of up to 64 R channels)
+__global__ void __launch_bounds__(kScanThreads)
+delta_scan_kernel(const float* __restrict__ qk, const float* __restrict__ kq, const float* __restrict__ f,
+                  const float* __restrict__ beta, const T* __restrict__ v, float* __restrict__ state, long long state_stride,
+                  const int* __restrict__ seg_q_start, const int* __restrict__ seg_q_len, const int* __restrict__ state_slots,
+                  float* __restrict__ y, int tokens, int heads, int groups, int dp, int p_dim) {
+    constexpr int kRow = 64 * R;                             // a token's k (q, f) in shared memory: DP channels and zeros
+    constexpr int kFours = kScanTokens * kRow / 4 / kScanThreads;      // groups of four of each that a thread stages: R
+    __shared__ __align__(16) float q_s[kScanTokens * kRow], k_s[kScanTokens * kRow], f_s[kScanTokens * kRow];
+    __shared__ float v_s[kScanTokens * kScanCols];
+    __shared__ float beta_s[kScanTokens], kq_s[kScanTokens];
+    const int h = blockIdx.x, seg = blockIdx.y, p0 = blockIdx.z * kScanCols;
+    const int q_len = seg_q_len[seg], q_start = seg_q_start[seg];
+    if (q_len <= 0) return;
+    const int tid = threadIdx.x, lane = tid % kWave, wave = tid / kWave;
+    const int sl = lane % kScanLanes, col = wave * (kWave / kScanLanes) + lane / kScanLanes;
+    const int p = p0 + col;
+    const bool live = p < p_dim;
+    const int g = h / (heads / groups);
+    float* s_col = state + static_cast<size_t>(state_slots[seg]) * state_stride + (static_cast<size_t>(h) * p_dim + p) * dp;
+    float4 s[R];
+#pragma unroll
+    for (int j = 0; j < R; ++j) {
+        const int i = 64 * j + 4 * sl;
+        s[j] = live && i < dp ? *reinterpret_cast<const float4*>(s_col + i) : make_float4(0.f, 0.f, 0.f, 0.f);
+    }
+    const size_t q_width = static_cast<size_t>(groups) * dp, f_width = static_cast<size_t>(heads) * dp;
+    const size_t k_plane = static_cast<size_t>(tokens) * q_width;
+    float4 q_r[kFours], k_r[kFours], f_r[kFours];
+    float v_r = 0.f, beta_r = 0.f, kq_r = 0.f;
+    const int vt = tid / kScanCols, vc = tid % kScanCols;    // (16 tokens of 16 columns: one value a thread)
+    auto fetch = [&](int t0) {
+        const int count = min(kScanTokens, q_len - t0);
+        const size_t first = static_cast<size_t>(q_start + t0);
+#pragma unroll
+        for (int u = 0; u < kFours; ++u) {
+            const int four = tid + kScanThreads * u;
+            const int t = four / (kRow / 4), i = four % (kRow / 4) * 4;
+            q_r[u] = k_r[u] = f_r[u] = make_float4(0.f, 0.f, 0.f, 0.f);
+            if (t < count && i < dp) {
+                const float* at = qk + (first + t) * q_width + static_cast<size_t>(g) * dp + i;
+                q_r[u] = *reinterpret_cast<const float4*>(at);
+                k_r[u] = *reinterpret_cast<const float4*>(at + k_plane);
+                f_r[u] = *reinterpret_cast<const float4*>(f + (first + t) * f_width + static_cast<size_t>(h) * dp + i);
+            }
+        }
+        v_r = vt < count && p0 + vc < p_dim ? to_float(v[(first + vt) * heads * p_dim + static_cast<size_t>(h) * p_dim + p0 + vc]) : 0.f;
+        if (tid < count) {
+            beta_r = beta[(first + tid) * heads + h];
+            kq_r = kq[(first + tid) * groups + g];
+        }
+    };
+    auto place = [&]() {
+#pragma unroll
+        for (int u = 0; u < kFours; ++u) {
+            const int four = tid + kScanThreads * u;
+            reinterpret_cast<float4*>(q_s)[four] = q_r[u];
+            reinterpret_cast<float4*>(k_s)[four] = k_r[u];
+            reinterpret_cast<float4*>(f_s)[four] = f_r[u];
+        }
+        v_s[tid] = v_r;
+        if (tid < kScanTokens) {
+            beta_s[tid] = beta_r;
+            kq_s[tid] = kq_r;
+        }
+    };
+    float kept = 0.f;                                        // lane sl of a column keeps the result of token sl of the 16
+    auto token = [&](int t) {
+        float4 kt[R];
+        float seen[2] = {0.f, 0.f}, read[2] = {0.f, 0.f};    // two chains each
+#pragma unroll
+        for (int j = 0; j < R; ++j) {
+            const int at = t * kRow + 64 * j + 4 * sl;
+            kt[j] = *reinterpret_cast<const float4*>(k_s + at);
+            const float4 qt = *reinterpret_cast<const float4*>(q_s + at), ft = *reinterpret_cast<const float4*>(f_s + at);
+            s[j].x *= ft.x;
+            s[j].y *= ft.y;
+            s[j].z *= ft.z;
+            s[j].w *= ft.w;
+            seen[0] = fmaf(s[j].x, kt[j].x, seen[0]);
+            seen[1] = fmaf(s[j].y, kt[j].y, seen[1]);
+            seen[0] = fmaf(s[j].z, kt[j].z, seen[0]);
+            seen[1] = fmaf(s[j].w, kt[j].w, seen[1]);
+            read[0] = fmaf(s[j].x, qt.x, read[0]);
+            read[1] = fmaf(s[j].y, qt.y, read[1]);
+            read[0] = fmaf(s[j].z, qt.z, read[0]);
+            read[1] = fmaf(s[j].w, qt.w, read[1]);
+        }
+        const float u = beta_s[t] * (v_s[t * kScanCols + col] - row_sum(seen[0] + seen[1]));
+        const float o = fmaf(u, kq_s[t], row_sum(read[0] + read[1]));
+#pragma unroll
+        for (int j = 0; j < R; ++j) {
+            s[j].x = fmaf(kt[j].x, u, s[j].x);
+            s[j].y = fmaf(kt[j].y, u, s[j].y);
+            s[j].z = fmaf(kt[j].z, u, s[j].z);
+            s[j].w = fmaf(kt[j].w, u, s[j].w);
+        }
+        if (sl == t) kept = o;
+    };
+    fetch(0);
+    for (int t0 = 0; t0 < q_len; t0 += kScanTokens) {
+        const int count = min(kScanTokens, q_len - t0);
+        place();
+        __syncthreads();
+        if (t0 + kScanTokens < q_len) fetch(t0 + kScanTokens);
+        if (count == kScanTokens) {
+#pragma unroll
+            for (int t = 0; t < kScanTokens; ++t) token(t);
+        } else {
+            for (int t = 0; t < count; ++t) token(t);
+        }
+        if (live && sl < count)
+            y[static_cast<size_t>(q_start + t0 + sl) * heads * p_dim + static_cast<size_t>(h) * p_dim + p] = kept;
+        __syncthreads();                                     // the 16 tokens are read out
+    }
+    if (live) {
+#pragma unroll
+        for (int j = 0; j < R; ++j) {
+            const int i = 64 * j + 4 * sl;
+            if (i < dp) *reinterpret_cast<float4*>(s_col + i) = s[j];
+        }
+    }
+}
+
+WLLM_API int wllm_delta_scan(const float* qk, const float* kq, const float* f, const float* beta, const void* v, float* state,
+                             long long state_stride, const int* seg_q_start, const int* seg_q_len, const int* state_slots, float* y,
+                             int is_bf16, int tokens, int segments, int heads, int groups, int d, int p_dim, hipStream_t stream) {
+    if (tokens <= 0 || segments <= 0) return 0;
+    if (heads <= 0 || groups <= 0 || heads % groups || d <= 0 || d > 256 || p_dim <= 0 || segments > 65535 ||
+        (p_dim + kScanCols - 1) / kScanCols > 65535 || state_stride % 4 || reinterpret_cast<uintptr_t>(state) % 16)
+        return -1;
+    const int dp = (d + 3) / 4 * 4;
+    const dim3 grid(heads, segments, (p_dim + kScanCols - 1) / kScanCols);
+#define LAUNCH(T, R)                                                                                                   \
+    delta_scan_kernel<T, R><<<grid, kScanThreads, 0, stream>>>(qk, kq, f, beta, static_cast<const T*>(v), state, state_stride, \
+                                                               seg_q_start, seg_q_len, state_slots, y, tokens, heads, groups, dp, \
+                                                               p_dim)
+#define LAUNCH_R(T)                    \
+    if (dp <= 64) LAUNCH(T, 1);        \
+    else if (dp <= 128) LAUNCH(T, 2);  \
+    else if (dp <= 192) LAUNCH(T, 3);  \
+    else LAUNCH(T, 4);
+    if (is_bf16) { LAUNCH_R(bf16) } else { LAUNCH_R(float) }
+#undef LAUNCH_R
+#undef LAUNCH
+    return launch_status();
+}

@@ -492,3 +492,55 @@ WLLM_API int wllm_gated_activation(const void* gate_up, void* out, int is_bf16, 
 #undef LAUNCH
     return launch_status();
 }
+
+// ---- an activation alone: out[i] = act(in[i]) (the feed-forward without a gate, behind a product of many rows);
+// out may be in ----
+template <typename T, int ACT>
+__global__ void __launch_bounds__(256) activation_kernel(const T* __restrict__ in, T* __restrict__ out, long long total) {
+    const long long stride = static_cast<long long>(gridDim.x) * blockDim.x;
+    for (long long i = static_cast<long long>(blockIdx.x) * blockDim.x + threadIdx.x; i < total; i += stride)
+        out[i] = from_float<T>(activate_single<ACT>(to_float(in[i])));
+}
+
+// eight bfloat16 a 16-byte access
+template <int ACT>
+__global__ void __launch_bounds__(256)
+activation_bf16x8_kernel(const bf16* __restrict__ in, bf16* __restrict__ out, long long vecs) {
+    const long long stride = static_cast<long long>(gridDim.x) * blockDim.x;
+    for (long long i = static_cast<long long>(blockIdx.x) * blockDim.x + threadIdx.x; i < vecs; i += stride) {
+        const uint4 v = load_streamed(in + i * 8);
+        const uint32_t w[4] = {v.x, v.y, v.z, v.w};
+        uint32_t o[4];
+#pragma unroll
+        for (int k = 0; k < 4; ++k)
+            o[k] = pack2_bf16(activate_single<ACT>(__uint_as_float(w[k] << 16)),
+                              activate_single<ACT>(__uint_as_float(w[k] & 0xffff0000u)));
+        *reinterpret_cast<uint4*>(out + i * 8) = make_uint4(o[0], o[1], o[2], o[3]);
+    }
+}
+
+WLLM_API int wllm_activation(const void* in, void* out, int is_bf16, int activation, long long total, hipStream_t stream) {
+    if (total <= 0) return 0;
+    if (activation < 0 || activation >= kSingleActivations) return -1;
+    const bool vec = is_bf16 && total % 8 == 0 && reinterpret_cast<uintptr_t>(in) % 16 == 0 &&
+                     reinterpret_cast<uintptr_t>(out) % 16 == 0;
+    long long blocks = ((vec ? total / 8 : total) + 255) / 256;
+    if (blocks > 16384) blocks = 16384;
+#define LAUNCH(ACT)                                                                                                    \
+    if (vec)                                                                                                           \
+        activation_bf16x8_kernel<ACT><<<static_cast<int>(blocks), 256, 0, stream>>>(static_cast<const bf16*>(in),      \
+                                                                                    static_cast<bf16*>(out), total / 8); \
+    else if (is_bf16)                                                                                                  \
+        activation_kernel<bf16, ACT><<<static_cast<int>(blocks), 256, 0, stream>>>(static_cast<const bf16*>(in),       \
+                                                                                   static_cast<bf16*>(out), total);    \
+    else                                                                                                               \
+        activation_kernel<float, ACT><<<static_cast<int>(blocks), 256, 0, stream>>>(static_cast<const float*>(in),     \
+                                                                                    static_cast<float*>(out), total)
+    switch (activation) {
+        case kActGeluTanh: LAUNCH(kActGeluTanh); break;
+        case kActSilu: LAUNCH(kActSilu); break;
+        default: LAUNCH(kActSquaredRelu); break;
+    }
+#undef LAUNCH
+    return launch_status();
+}

@@ -333,6 +333,8 @@ WLLM_API int wllm_gemm_skinny(const void* x, const void* w, int tiled, void* out
 // A wavefront streams 16 gate rows and the 16 up rows that belong to them; both results land
 // in the same lanes, so the activation and the product are made in registers and only [M, I]
 // is written.
+// With the paired squared relu there is no gate: w is one matrix of 2I rows, out[M, 2I] = relu(x . w^T)^2, whose two
+// halves of the columns are the two streams.
 
 // A workgroup is TPW tiles of 16 gate rows (with their up rows) times 2 halves of the K axis; the
 // halves are added through shared memory in a fixed order before the activation.  A workgroup is 2
@@ -528,27 +530,37 @@ gemm_skinny_gated_kernel(const bf16* __restrict__ x, NormOnLoad norm, const bf16
     for (int t = 0; t < MT; ++t) {
         const int m = t * 16 + i;
         if (m >= M) continue;
-        float4_t r;
+        constexpr bool kPair = GATE == kGatePairSquaredRelu;
+        float4_t r, r2;
 #pragma unroll
         for (int v = 0; v < 4; ++v) {
             const float gate = accg[t][v] + red[t * 8 + v], upv = accu[t][v] + red[t * 8 + 4 + v];
-            r[v] = gate_product<GATE>(gate, upv, shape);
+            if (kPair) {
+                r[v] = squared_relu(gate);
+                r2[v] = squared_relu(upv);
+            } else {
+                r[v] = gate_product<(kPair ? 0 : GATE)>(gate, upv, shape);
+            }
         }
         bf16* o = out + static_cast<size_t>(m) * out_stride + n;     // out may be a band of columns of a wider buffer
         if (n + 3 < inter && (inter % 4 == 0) && (out_stride % 4 == 0)) {
             store4<bf16>(o, r);
+            if (kPair) store4<bf16>(o + inter, r2);
         } else {
 #pragma unroll
             for (int v = 0; v < 4; ++v)
-                if (n + v < inter) o[v] = from_float<bf16>(r[v]);
+                if (n + v < inter) {
+                    o[v] = from_float<bf16>(r[v]);
+                    if (kPair) o[inter + v] = from_float<bf16>(r2[v]);
+                }
         }
     }
 }
 
 static int gated_launch(const void* x, NormOnLoad norm, bool with_norm, const void* w, int tiled, void* out, int M,
                         int inter, int K, int gate, GateShape shape, int chunk, int out_stride, hipStream_t stream) {
-    if (out_stride < inter) return -1;
-    if (M < 1 || M > 64 || K % 64 != 0 || chunk % 32 != 0 || gate < 0 || gate >= kGates) return -1;
+    if (out_stride < (gate == kGatePairSquaredRelu ? 2 * inter : inter)) return -1;
+    if (M < 1 || M > 64 || K % 64 != 0 || chunk % 32 != 0 || gate < 0 || gate >= (with_norm ? kGates : kPairedGates)) return -1;
     const int mt = (M + 15) / 16;
     if (chunk > K / 2) chunk = K / 2;
     // the norm on load: at most 16 rows, whole chunks of 256 keys
@@ -598,7 +610,7 @@ static int gated_launch(const void* x, NormOnLoad norm, bool with_norm, const vo
     if (with_norm) {
         WLLM_BY_GATE(gate, LAUNCH_N(GATE))
     } else {
-        WLLM_BY_GATE(gate, BY_MT(GATE))
+        WLLM_BY_PAIRED_GATE(gate, BY_MT(GATE))
     }
 #undef BY_MT
 #undef LAUNCH_N

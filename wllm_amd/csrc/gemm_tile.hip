@@ -168,22 +168,37 @@ gemm_tile_kernel(const bf16* __restrict__ x, const bf16* __restrict__ w, bf16* _
             for (int a = 0; a < 2; ++a) {
                 const int n = n_base + wn * 32 + 16 * a + 4 * g;
                 if (n >= N) continue;
-                float r[4];
+                // (the paired squared relu: no gate, the two streams are the two halves of a row of 2 N columns)
+                constexpr bool kPair = GATED == kGatePairSquaredRelu + 1;
+                float r[4], r2[4];
 #pragma unroll
                 for (int v = 0; v < 4; ++v) {
                     const float gate = acc[a][b][v], up = acc[a + 2][b][v];
-                    r[v] = gate_product<(GATED > 0 ? GATED - 1 : 0)>(gate, up, shape);
+                    if (kPair) {
+                        r[v] = squared_relu(gate);
+                        r2[v] = squared_relu(up);
+                    } else {
+                        r[v] = gate_product<(GATED > 0 && !kPair ? GATED - 1 : 0)>(gate, up, shape);
+                    }
                 }
-                bf16* o = out + static_cast<size_t>(m) * N + n;
+                bf16* o = out + static_cast<size_t>(m) * (kPair ? 2 * N : N) + n;
                 if (n + 3 < N && N % 4 == 0) {
                     uint2 p;
                     p.x = pack2_bf16(r[0], r[1]);
                     p.y = pack2_bf16(r[2], r[3]);
                     *reinterpret_cast<uint2*>(o) = p;
+                    if (kPair) {
+                        p.x = pack2_bf16(r2[0], r2[1]);
+                        p.y = pack2_bf16(r2[2], r2[3]);
+                        *reinterpret_cast<uint2*>(o + N) = p;
+                    }
                 } else {
 #pragma unroll
                     for (int v = 0; v < 4; ++v)
-                        if (n + v < N) o[v] = from_float<bf16>(r[v]);
+                        if (n + v < N) {
+                            o[v] = from_float<bf16>(r[v]);
+                            if (kPair) o[N + v] = from_float<bf16>(r2[v]);
+                        }
                 }
             }
         } else {
@@ -220,12 +235,12 @@ gemm_tile_kernel(const bf16* __restrict__ x, const bf16* __restrict__ w, bf16* _
 }
 
 // out[M, N] = x . w^T (gated 0, w [N, K]), or the gated product (gated = 1 + the gate's number, with limit, slope and
-// shift for the clamped swish; w [2N, K], gate rows first).  splits > 1 (plain only): `out` is null and `partial` float32
+// shift for the clamped swish; w [2N, K], gate rows first; with the paired squared relu out [M, 2N] = relu(x . w^T)^2).  splits > 1 (plain only): `out` is null and `partial` float32
 // [splits, M, N] takes the pieces' sums.  K must be a multiple of 64 * splits and the operands smaller
 // than 4 GiB.  Returns 0, a HIP error code, or -1 for sizes it does not take.
 WLLM_API int wllm_gemm_tile(const void* x, const void* w, void* out, float* partial, int M, int N, int K, int splits,
                             int gated, float limit, float slope, float shift, hipStream_t stream) {
-    if (M < 1 || N < 1 || K < kStageKeys || splits < 1 || K % (kStageKeys * splits) != 0 || gated < 0 || gated > kGates)
+    if (M < 1 || N < 1 || K < kStageKeys || splits < 1 || K % (kStageKeys * splits) != 0 || gated < 0 || gated > kPairedGates)
         return -1;
     if ((splits > 1) != (partial != nullptr) || (splits == 1 && out == nullptr) || (splits > 1 && gated != 0)) return -1;
     const size_t w_rows = static_cast<size_t>(gated ? 2 : 1) * N;
@@ -267,7 +282,7 @@ WLLM_API int wllm_gemm_tile(const void* x, const void* w, void* out, float* part
     if (deep) LAUNCH(GATED, 4);         \
     else LAUNCH(GATED, 2)
     if (gated == 0) { BY_STAGES(0); }
-    else { WLLM_BY_GATE(gated - 1, BY_STAGES(GATE + 1)) }
+    else { WLLM_BY_PAIRED_GATE(gated - 1, BY_STAGES(GATE + 1)) }
 #undef BY_STAGES
 #undef LAUNCH
     return launch_status();

@@ -26,6 +26,7 @@ template <typename T> struct alignas(4 * sizeof(T)) Four { T v[4]; };
 //      (interleaved) or (j, j + rotary_dim / 2); sine and cosine are multiplied by rot_scale;
 //   4. with norm_eps >= 0 the head is divided by sqrt(sum of its squares / norm_dim + norm_eps) (norm_dim is
 //      head_dim, or less where the last elements of a head are padding that is always zero);
+//   4b. with temp_every > 0 a query head is multiplied by 1 + temp_coef * ln(floor((position + 1) / temp_every) + 1);
 //   5. it is written back to the row, and a key head to the cache's keys.
 // Value heads of their own and the rest of the row take step 1 only.  Keys lie in the cache as
 // [page_size, head_dim], values transposed as [head_dim, page_size].
@@ -44,7 +45,8 @@ head_prepare_kernel(T* __restrict__ rows, int row_width, const float* __restrict
                     const float* __restrict__ inv_freq, const int* __restrict__ slots, T* __restrict__ cache,
                     long long num_pages, int num_heads, int num_kv_heads, int head_dim, int rotary_dim,
                     int interleaved, float norm_eps, int norm_dim, int values_are_keys, int page_size, int head_pieces,
-                    const float* __restrict__ pre_q, const float* __restrict__ pre_k, float pre_eps, float rot_scale) {
+                    const float* __restrict__ pre_q, const float* __restrict__ pre_k, float pre_eps, float rot_scale,
+                    float temp_coef, int temp_every) {
     __shared__ float staged[kPrepareWaves][FOUR ? 1 : kPrepareMaxHead];
     const int token = blockIdx.x;
     const int lane = threadIdx.x % kWave, wave = threadIdx.x / kWave;
@@ -96,6 +98,8 @@ head_prepare_kernel(T* __restrict__ rows, int row_width, const float* __restrict
     const int base = head * head_dim;
     const int kvh = head - num_heads;                 // >= 0: a key head
     const int half = rotary_dim / 2;
+    float temperature = 1.f;
+    if (temp_every > 0 && kvh < 0) temperature = 1.f + temp_coef * logf(static_cast<float>((positions[token] + 1) / temp_every) + 1.f);
     if (FOUR) {
         const int e = 4 * lane;
         float v[4] = {0.f, 0.f, 0.f, 0.f};
@@ -162,6 +166,7 @@ head_prepare_kernel(T* __restrict__ rows, int row_width, const float* __restrict
             const float ss = wave_sum(v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3]);
             inv = rsqrtf(ss / static_cast<float>(norm_dim) + norm_eps);
         }
+        inv *= temperature;
         if (live) {
             Four<T> r;
 #pragma unroll
@@ -220,6 +225,7 @@ head_prepare_kernel(T* __restrict__ rows, int row_width, const float* __restrict
     }
     float inv = 1.f;
     if (norm_eps >= 0.f) inv = rsqrtf(wave_sum(ss) / static_cast<float>(norm_dim) + norm_eps);
+    inv *= temperature;
 #pragma unroll
     for (int k = 0; k < kPerLane; ++k) {
         const int e = lane + k * kWave;
@@ -238,12 +244,13 @@ WLLM_API int wllm_head_prepare(void* rows, int is_bf16, int row_width, const flo
                                const float* inv_freq, const int* slots, void* cache, long long num_pages, int n,
                                int num_heads, int num_kv_heads, int head_dim, int rotary_dim, int interleaved,
                                float norm_eps, int norm_dim, int values_are_keys, int page_size, const float* pre_q,
-                               const float* pre_k, float pre_eps, float rot_scale, hipStream_t stream) {
+                               const float* pre_k, float pre_eps, float rot_scale, float temp_coef, int temp_every,
+                               hipStream_t stream) {
     if (pre_eps >= 0.f && (pre_q == nullptr || (pre_k == nullptr && num_kv_heads > 0))) return -1;
     const int heads = num_heads + (values_are_keys ? 1 : 2) * num_kv_heads;
     if (head_dim <= 0 || head_dim > kPrepareMaxHead || rotary_dim < 0 || rotary_dim > head_dim || rotary_dim % 2 != 0 ||
         row_width < heads * head_dim || num_heads < 0 || num_kv_heads < 0 || page_size <= 0 || bias_width < 0 ||
-        bias_width > row_width || (bias == nullptr && bias_width != 0) || norm_dim <= 0 || norm_dim > head_dim)
+        bias_width > row_width || (bias == nullptr && bias_width != 0) || norm_dim <= 0 || norm_dim > head_dim || temp_every < 0)
         return -1;
     if (inv_freq == nullptr && rotary_dim != 0) return -1;
     if (n <= 0) return 0;
@@ -262,7 +269,8 @@ WLLM_API int wllm_head_prepare(void* rows, int is_bf16, int row_width, const flo
     head_prepare_kernel<T, FOUR><<<grid, kWave * kPrepareWaves, 0, stream>>>(                                       \
         static_cast<T*>(rows), row_width, parts, splits, static_cast<size_t>(split_stride), bias, bias_width, positions, \
         inv_freq, slots, static_cast<T*>(cache), num_pages, num_heads, num_kv_heads, head_dim, rotary_dim, interleaved, \
-        norm_eps, norm_dim, values_are_keys, page_size, head_pieces, pre_q, pre_k, pre_eps, rot_scale)
+        norm_eps, norm_dim, values_are_keys, page_size, head_pieces, pre_q, pre_k, pre_eps, rot_scale, temp_coef, \
+        temp_every)
     if (is_bf16) {
         if (four) LAUNCH(bf16, true); else LAUNCH(bf16, false);
     } else {

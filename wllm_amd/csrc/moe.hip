@@ -1,9 +1,10 @@
 // A mixture of gated feed-forward experts on a flat batch of tokens: the router, the plan that sorts a
 // step's (token, chosen expert) pairs by expert, and the two grouped products on the matrix cores.
 //
-//   router   z = W_r x (float32), s = softmax(z) over all experts (or, `scoring` 1, s = sigmoid(z) of each); only experts of the `keep` best of
-//            `groups` equal groups of neighbours (a group's score: its largest s) may be chosen; the `top`
-//            allowed experts with the largest s are chosen, weights s / (sum of the chosen + eps) (or, `normalize` 0, s itself)
+//   router   z = W_r x (float32), s = softmax(z) over all experts (or, `scoring` 1, s = sigmoid(z) of each); what is compared
+//            is c = s + correction (none: s); only experts of the `keep` best of `groups` equal groups of neighbours (a
+//            group's score: its largest c, or the sum of its two largest) may be chosen; the `top` allowed experts with the
+//            largest c are chosen, weights s / (sum of the chosen + eps) (or, `normalize` 0, s itself)
 //   plan     an assignment is a = token * top + slot.  The assignments of one expert lie together, in
 //            tiles of R rows (16, 32, 64 or 128; the last tile of an expert padded with -1):
 //            plan[0] = tiles in use; plan[1 + t] = expert of tile t; plan[1 + max_tiles + R t + r] = a or -1
@@ -26,21 +27,27 @@ constexpr int kMoeMaxExperts = 256;
 
 // ---- the router: one workgroup a token.  The four wavefronts share the experts' dot products (a lane sums its
 // columns in ascending order, the lanes are added in the butterfly's order: the same bits whatever the batch);
-// then the first wavefront, a lane holding the experts lane, lane + 64, ..., takes the softmax, shuts the groups
-// out and picks the top, every choice a maximum over the wavefront and, among equals, the lowest index. ----
+// then the first wavefront, a lane holding the experts lane, lane + 64, ..., takes the scores, shuts the groups
+// out and picks the top, every choice a maximum over the wavefront and, among equals, the lowest index.
+// What decides the choice (of groups and of experts) is score + correction (no correction: the score); the weights
+// come of the scores alone.  A group's score is the sum of its `group_best` (1 or 2) largest choice scores.  With
+// `gates` the router has one more row, behind the experts': the sigmoid of its product is left in gates[token]. ----
 constexpr int kRoutePer = kMoeMaxExperts / kWave;        // experts a lane holds
 
 __device__ __forceinline__ int wave_lowest(int v) { return -static_cast<int>(wave_max(-static_cast<float>(v))); }
 
 template <typename T>
 __global__ void __launch_bounds__(256)
-moe_route_kernel(const T* __restrict__ x, const float* __restrict__ router, int* __restrict__ ids, float* __restrict__ weights,
-                 int tokens, int width, int experts, int top, int groups, int keep, float eps, int scoring, int normalize) {
-    __shared__ float z_s[kMoeMaxExperts];
+moe_route_kernel(const T* __restrict__ x, const float* __restrict__ router, const float* __restrict__ correction,
+                 int* __restrict__ ids, float* __restrict__ weights, float* __restrict__ gates, int tokens, int width,
+                 int experts, int top, int groups, int keep, int group_best, float eps, int scoring, int normalize) {
+    __shared__ float z_s[kMoeMaxExperts + 1];            // products; from the first wavefront's second pass on, scores
+    __shared__ float c_s[kMoeMaxExperts];                // choice scores
     const int wave = threadIdx.x / kWave, lane = threadIdx.x % kWave;
     const int token = blockIdx.x;
     const T* xr = x + static_cast<size_t>(token) * width;
-    for (int e = wave; e < experts; e += 4) {
+    const int products = experts + (gates ? 1 : 0);
+    for (int e = wave; e < products; e += 4) {
         const float* w = router + static_cast<size_t>(e) * width;
         float dot = 0.f;
         if (width % 4 == 0) {
@@ -60,58 +67,66 @@ moe_route_kernel(const T* __restrict__ x, const float* __restrict__ router, int*
     }
     __syncthreads();
     if (wave != 0) return;
-    // softmax over all experts
+    if (gates && lane == 0) gates[token] = 1.f / (1.f + expf(-z_s[experts]));
+    // the scores: a sigmoid of each, or the softmax over all experts
     float sc[kRoutePer];
-    float mx = -INFINITY;
 #pragma unroll
-    for (int j = 0; j < kRoutePer; ++j) {
-        const int e = lane + kWave * j;
-        sc[j] = e < experts ? z_s[e] : -INFINITY;
-        mx = fmaxf(mx, sc[j]);
-    }
-    mx = wave_max(mx);
-    float sum = 0.f;
+    for (int j = 0; j < kRoutePer; ++j) sc[j] = lane + kWave * j < experts ? z_s[lane + kWave * j] : -INFINITY;
     if (scoring == 1) {
-        // a score of each expert by itself: in the terms of the softmax's code below, exp(z - mx) / sum with mx = 0
-        // and sum = 1 would not do (it overflows), so the sigmoid is written into sc and z_s as it is
-        __builtin_amdgcn_wave_barrier();
 #pragma unroll
-        for (int j = 0; j < kRoutePer; ++j) {
-            const int e = lane + kWave * j;
-            sc[j] = e < experts ? 1.f / (1.f + expf(-sc[j])) : 0.f;
-            if (e < experts) z_s[e] = sc[j];
-        }
-        __builtin_amdgcn_wave_barrier();
-        asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
-        sum = 1.f;
+        for (int j = 0; j < kRoutePer; ++j) sc[j] = 1.f / (1.f + expf(-sc[j]));
     } else {
+        float mx = sc[0];
+#pragma unroll
+        for (int j = 1; j < kRoutePer; ++j) mx = fmaxf(mx, sc[j]);
+        mx = wave_max(mx);
+        float sum = 0.f;
 #pragma unroll
         for (int j = 0; j < kRoutePer; ++j) {
             sc[j] = lane + kWave * j < experts ? expf(sc[j] - mx) : 0.f;
             sum += sc[j];
         }
         sum = wave_sum(sum);
-    }
-    // a score that may still be chosen is >= 0; one that may not is -1
 #pragma unroll
-    for (int j = 0; j < kRoutePer; ++j) sc[j] = lane + kWave * j < experts ? sc[j] / sum : -1.f;
+        for (int j = 0; j < kRoutePer; ++j) sc[j] /= sum;
+    }
+    // what may not be chosen (any more) is minus infinity; every lane reads what others leave in shared memory
+#pragma unroll
+    for (int j = 0; j < kRoutePer; ++j) {
+        const int e = lane + kWave * j;
+        if (e < experts) {
+            z_s[e] = sc[j];
+            sc[j] += correction ? correction[e] : 0.f;
+            c_s[e] = sc[j];
+        } else {
+            sc[j] = -INFINITY;
+        }
+    }
+    __builtin_amdgcn_wave_barrier();
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
     if (keep < groups) {
         const int per = experts / groups;
-        float gs[kRoutePer];                     // the scores of the groups lane, lane + 64, ...: their largest member's
+        float gs[kRoutePer];                     // the scores of the groups lane, lane + 64, ...
         bool allowed[kRoutePer];
 #pragma unroll
         for (int j = 0; j < kRoutePer; ++j) {
             const int g = lane + kWave * j;
-            gs[j] = -1.f;
+            gs[j] = -INFINITY;
             allowed[j] = false;
-            if (g < groups)
-                for (int m = 0; m < per; ++m)
-                    gs[j] = fmaxf(gs[j], scoring == 1 ? z_s[g * per + m] : expf(z_s[g * per + m] - mx) / sum);
+            if (g < groups) {
+                float first = -INFINITY, second = -INFINITY;
+                for (int m = 0; m < per; ++m) {
+                    const float c = c_s[g * per + m];
+                    second = fmaxf(second, fminf(first, c));
+                    first = fmaxf(first, c);
+                }
+                gs[j] = group_best == 2 && per > 1 ? first + second : first;
+            }
         }
         for (int pick = 0; pick < keep; ++pick) {
-            float best = -1.f;
+            float best = gs[0];
 #pragma unroll
-            for (int j = 0; j < kRoutePer; ++j) best = fmaxf(best, gs[j]);
+            for (int j = 1; j < kRoutePer; ++j) best = fmaxf(best, gs[j]);
             best = wave_max(best);
             int which = kMoeMaxExperts;
 #pragma unroll
@@ -120,34 +135,35 @@ moe_route_kernel(const T* __restrict__ x, const float* __restrict__ router, int*
             which = wave_lowest(which);
 #pragma unroll
             for (int j = 0; j < kRoutePer; ++j) {
-                if (lane + kWave * j == which) gs[j] = -1.f;
+                if (lane + kWave * j == which) gs[j] = -INFINITY;
                 if ((lane + kWave * j) / per == which) allowed[j] = true;
             }
         }
 #pragma unroll
         for (int j = 0; j < kRoutePer; ++j)
-            if (!allowed[j]) sc[j] = -1.f;
+            if (!allowed[j]) sc[j] = -INFINITY;
     }
     float chosen_sum = 0.f;
     int* id = ids + static_cast<size_t>(token) * top;
     float* wt = weights + static_cast<size_t>(token) * top;
     for (int slot = 0; slot < top; ++slot) {
-        float best = -1.f;
+        float best = sc[0];
 #pragma unroll
-        for (int j = 0; j < kRoutePer; ++j) best = fmaxf(best, sc[j]);
+        for (int j = 1; j < kRoutePer; ++j) best = fmaxf(best, sc[j]);
         best = wave_max(best);
         int which = kMoeMaxExperts;
 #pragma unroll
         for (int j = kRoutePer - 1; j >= 0; --j)
             if (sc[j] == best) which = lane + kWave * j;
-        which = wave_lowest(which);
+        which = min(wave_lowest(which), experts - 1);        // (a token whose scores are no numbers still names an expert)
 #pragma unroll
         for (int j = 0; j < kRoutePer; ++j)
-            if (lane + kWave * j == which) sc[j] = -1.f;
-        chosen_sum += best;
+            if (lane + kWave * j == which) sc[j] = -INFINITY;
+        const float score = z_s[which];
+        chosen_sum += score;
         if (lane == 0) {
             id[slot] = which;
-            wt[slot] = best;
+            wt[slot] = score;
         }
     }
     if (lane == 0 && normalize) {
@@ -156,20 +172,23 @@ moe_route_kernel(const T* __restrict__ x, const float* __restrict__ router, int*
     }
 }
 
-WLLM_API int wllm_moe_route(const void* x, const float* router, int* ids, float* weights, int is_bf16, int tokens, int width,
-                            int experts, int top, int groups, int keep, float eps, int scoring, int normalize,
-                            hipStream_t stream) {
+// `correction` float32 [experts] or null; `gates` float32 [tokens] or null (then `router` has experts + 1 rows).
+WLLM_API int wllm_moe_route(const void* x, const float* router, const float* correction, int* ids, float* weights, float* gates,
+                            int is_bf16, int tokens, int width, int experts, int top, int groups, int keep, int group_best,
+                            float eps, int scoring, int normalize, hipStream_t stream) {
     if (tokens <= 0) return 0;
-    if (scoring < 0 || scoring > 1) return -1;
+    if (scoring < 0 || scoring > 1 || group_best < 1 || group_best > 2) return -1;
     if (experts <= 0 || experts > kMoeMaxExperts || groups <= 0 || experts % groups || keep <= 0 || keep > groups || top <= 0 ||
         top > keep * (experts / groups) || width <= 0)
         return -1;
     if (is_bf16)
-        moe_route_kernel<bf16><<<tokens, 256, 0, stream>>>(static_cast<const bf16*>(x), router, ids, weights, tokens, width,
-                                                           experts, top, groups, keep, eps, scoring, normalize);
+        moe_route_kernel<bf16><<<tokens, 256, 0, stream>>>(static_cast<const bf16*>(x), router, correction, ids, weights, gates,
+                                                           tokens, width, experts, top, groups, keep, group_best, eps, scoring,
+                                                           normalize);
     else
-        moe_route_kernel<float><<<tokens, 256, 0, stream>>>(static_cast<const float*>(x), router, ids, weights, tokens, width,
-                                                            experts, top, groups, keep, eps, scoring, normalize);
+        moe_route_kernel<float><<<tokens, 256, 0, stream>>>(static_cast<const float*>(x), router, correction, ids, weights, gates,
+                                                            tokens, width, experts, top, groups, keep, group_best, eps, scoring,
+                                                            normalize);
     return launch_status();
 }
 

@@ -1,5 +1,5 @@
 // The residual stream's general norm step, for layers that put a norm behind a sublayer as well as
-// before it:   x += norm_d(delta);   out = norm_o(x).
+// before it:   x = norm_s(scale * x + norm_d(delta + extra));   out = norm_o(x)   (scale 1, no norm_s and no extra as a rule).
 //
 // x float32 [n, H] is the stream.  delta, what a sublayer left (a tensor of the activation type or a
 // float32 stack of partial sums added in stack order), is normalised by a norm of its own before it is
@@ -10,11 +10,27 @@
 // activation type.  Everything is float32: means, variances as means of squared deviations (two
 // passes over a row held in shared memory), the sum.  One workgroup a row.
 //
+// `join` says how the sublayer's result meets the stream where it is not simply added: x is weighed before the sum
+// (`scale`), the sum passes a norm of its own (`norm_s`: a layer that norms the sum of stream and sublayer), and the
+// result may have a second term (`extra`, a tensor or a stack as delta is), whose rows are multiplied by a number a
+// row (`extra_scale`: an expert that every token uses, behind its gate).
+//
 // `conv` (a step in which every row is its request's one new token): out is not a norm of the new x but the new x
 // through a short convolution over time, out[c] = x[c] + sum_k w[k, c] * (the request's k-th carried row, the last tap
 // x itself), and the carried rows (float32 [taps - 1, H] from `carried_offset` of row state_slots[row] of `state`)
 // move up by one and take x: what `stream_conv` does for single tokens, in the launch that settles the stream.
 #include "common.h"
+
+struct NormJoin {
+    float scale;               // of x before the sum
+    int s_kind;                // the norm of the sum
+    const float* s_weight;
+    float s_eps, s_offset;
+    const void* extra;         // null: none
+    int extra_bf16, extra_splits;
+    size_t extra_stride;
+    const float* extra_scale;  // float32 [n], or null: 1
+};
 
 struct NormConv {
     const float* weight;       // [taps, H], a row a tap; null: no convolution
@@ -53,7 +69,7 @@ __global__ void __launch_bounds__(1024)
 norm_add_kernel(float* __restrict__ x, const TD* __restrict__ delta, int splits, size_t split_stride, int d_kind,
                 const float* __restrict__ d_weight, float d_eps, float d_offset, const int* __restrict__ rows,
                 TO* __restrict__ out, int o_kind, const float* __restrict__ o_weight, float o_eps, float o_offset,
-                int hidden, NormConv conv) {
+                int hidden, NormConv conv, NormJoin join) {
     extern __shared__ float row[];
     __shared__ float scratch[16];
     const int orow = blockIdx.x;
@@ -82,6 +98,13 @@ norm_add_kernel(float* __restrict__ x, const TD* __restrict__ delta, int splits,
             float d;
             if (sizeof(TD) == sizeof(float) && splits > 1) d = stack_sum(reinterpret_cast<const float*>(dr) + i, splits, split_stride);
             else d = to_float(dr[i]);
+            if (join.extra) {
+                const size_t at = static_cast<size_t>(irow) * hidden + i;
+                float e;
+                if (join.extra_bf16) e = to_float(static_cast<const bf16*>(join.extra)[at]);
+                else e = stack_sum(static_cast<const float*>(join.extra) + at, join.extra_splits, join.extra_stride);
+                d = fmaf(join.extra_scale ? join.extra_scale[irow] : 1.f, e, d);
+            }
             row[i] = d;
         }
         __syncthreads();
@@ -90,9 +113,18 @@ norm_add_kernel(float* __restrict__ x, const TD* __restrict__ delta, int splits,
         for (int i = threadIdx.x; i < hidden; i += blockDim.x) {
             float d = row[i];                       // this thread's own elements: no other thread writes them
             if (d_kind != kNormNone) d = (d - mean) * inv * (d_offset + d_weight[i]);
-            const float v = xr[i] + d;
-            if (!rows) xr[i] = v;
+            const float v = fmaf(join.scale, xr[i], d);
+            if (!rows && join.s_kind == kNormNone) xr[i] = v;
             row[i] = v;
+        }
+        if (join.s_kind != kNormNone) {
+            __syncthreads();
+            row_stats(row, hidden, join.s_kind, join.s_eps, scratch, mean, inv);
+            for (int i = threadIdx.x; i < hidden; i += blockDim.x) {
+                const float v = (row[i] - mean) * inv * (join.s_offset + join.s_weight[i]);
+                if (!rows) xr[i] = v;
+                row[i] = v;
+            }
         }
     } else {
         for (int i = threadIdx.x; i < hidden; i += blockDim.x) row[i] = xr[i];
@@ -153,11 +185,19 @@ WLLM_API int wllm_norm_add(float* x, const void* delta, int delta_type, int spli
                            const float* d_weight, float d_eps, float d_offset, const int* rows, void* out, int out_type,
                            int o_kind, const float* o_weight, float o_eps, float o_offset, int num_rows, int hidden,
                            const float* conv_weight, int conv_taps, float* conv_state, long long conv_state_stride,
-                           long long conv_carried_offset, const int* conv_state_slots, hipStream_t stream) {
+                           long long conv_carried_offset, const int* conv_state_slots, float x_scale, int s_kind,
+                           const float* s_weight, float s_eps, float s_offset, const void* extra, int extra_bf16,
+                           int extra_splits, long long extra_stride, const float* extra_scale, hipStream_t stream) {
     if (num_rows <= 0) return 0;
     if (conv_weight && (!out || rows || o_kind != kNormNone || conv_taps < 1 || conv_taps > 64 || !conv_state || !conv_state_slots))
         return -1;
     const NormConv conv{conv_weight, conv_state, conv_state_stride, conv_carried_offset, conv_state_slots, conv_taps};
+    if (s_kind < 0 || s_kind > 2 || (s_kind != kNormNone && !s_weight)) return -1;
+    // what joins the stream by a weight, a norm or a second term is a sublayer's result
+    if (!delta && (extra || s_kind != kNormNone || x_scale != 1.f)) return -1;
+    if (extra && extra_splits < 1) return -1;
+    const NormJoin join{x_scale, s_kind, s_weight, s_eps, s_offset, extra, extra_bf16, extra_splits,
+                        static_cast<size_t>(extra_stride), extra_scale};
     if (hidden <= 0 || hidden > 16384 || !x) return -1;
     if (d_kind < 0 || d_kind > 2 || o_kind < 0 || o_kind > 2) return -1;
     if (delta && d_kind != kNormNone && !d_weight) return -1;
@@ -175,7 +215,7 @@ WLLM_API int wllm_norm_add(float* x, const void* delta, int delta_type, int spli
     norm_add_kernel<TD, TO><<<num_rows, threads, smem, stream>>>(x, static_cast<const TD*>(delta), splits,            \
                                                               static_cast<size_t>(split_stride), d_kind, d_weight,   \
                                                               d_eps, d_offset, rows, static_cast<TO*>(out), o_kind,   \
-                                                              o_weight, o_eps, o_offset, hidden, conv)
+                                                              o_weight, o_eps, o_offset, hidden, conv, join)
     if (delta_type && out_type) LAUNCH(bf16, bf16);
     else if (delta_type) LAUNCH(bf16, float);
     else if (out_type) LAUNCH(float, bf16);

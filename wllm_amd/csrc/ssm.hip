@@ -7,6 +7,7 @@
 // A fresh request's row is all zeros, which is both "S starts at zero" and "zeros before the start".
 // Everything that enters the recurrence is float32: step sizes, decays, the state, the sums.
 #include "common.h"
+#include "short_conv.h"
 
 // ---- convolution: out[t, c] = silu(bias[c] + sum_k w[c, k] * in[t - (taps - 1) + k, c]), the inputs
 // before the segment's first token taken from the carried rows.  in is a band of a wider row. ----
@@ -29,28 +30,6 @@ causal_conv_kernel(const T* __restrict__ in, long long in_stride, const float* _
             acc = fmaf(weight[static_cast<size_t>(c) * taps + k], v, acc);
         }
         out[static_cast<size_t>(token) * channels + c] = from_float<T>(acc / (1.f + expf(-acc)));
-    }
-}
-
-// ---- after the convolution of a step: the carried rows take the segment's last taps - 1 inputs (of
-// a segment shorter than that, the carried rows move up).  Row j's new value comes from a row above
-// it or from the step's inputs, so a thread that walks j upwards never reads what it wrote. ----
-template <typename T>
-__global__ void __launch_bounds__(256)
-conv_carry_kernel(const T* __restrict__ in, long long in_stride, float* __restrict__ state, long long state_stride,
-                  long long carried_offset, const int* __restrict__ seg_q_start, const int* __restrict__ seg_q_len,
-                  const int* __restrict__ state_slots, int channels, int taps) {
-    const int seg = blockIdx.x;
-    const int q_len = seg_q_len[seg], q_start = seg_q_start[seg];
-    if (q_len <= 0) return;
-    float* carried = state + static_cast<size_t>(state_slots[seg]) * state_stride + carried_offset;
-    for (int c = blockIdx.y * blockDim.x + threadIdx.x; c < channels; c += gridDim.y * blockDim.x) {
-        for (int j = 0; j < taps - 1; ++j) {
-            const int src = q_len - (taps - 1) + j;
-            carried[static_cast<size_t>(j) * channels + c] =
-                src >= 0 ? to_float(in[static_cast<size_t>(q_start + src) * in_stride + c])
-                         : carried[static_cast<size_t>(j + q_len) * channels + c];
-        }
     }
 }
 

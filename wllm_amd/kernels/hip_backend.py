@@ -503,6 +503,27 @@ class HipBackend:
         self.linear(x, weight, scratch, tiles if x.dtype == torch.float32 else None)
         ops.call("gated_activation", scratch, out, activation)
 
+    def activated_linear(self, x, weight, out, name, tiles=None, paired_tiles=None):
+        self._on_gpu(x, weight, out, tiles, paired_tiles)
+        m, k = x.shape
+        n = weight.shape[0]
+        half = n // 2
+        # the kernels that make a gated product's two streams make the two halves of these columns
+        if name == "squared_relu" and n % 2 == 0 and x.dtype == torch.bfloat16:
+            number = len(ops.ACTIVATIONS) + 1
+            if self.skinny_takes(x.dtype, m, k) and k % 64 == 0 and out.data_ptr() % 8 == 0:
+                w, tiled = (paired_tiles, 1) if paired_tiles is not None else (weight, 0)
+                self._check(self.lib.wllm_gemm_skinny_gated(
+                    _ptr(x), _ptr(w), tiled, _ptr(out), m, half, k, number, 0.0, 0.0, 0.0, self.GATED_CHUNK[-(-m // 16)], n,
+                    self._stream()), "activated_linear (few rows, matrix cores)")
+                return
+            if 64 < m <= self.TILE_GATED_MAX_ROWS and k % 64 == 0 and max(m, n) * k * 2 < 2 ** 32:
+                self._check(self.lib.wllm_gemm_tile(_ptr(x), _ptr(weight), _ptr(out), None, m, half, k, 1, 1 + number, 0.0, 0.0,
+                                                    0.0, self._stream()), "activated_linear (tiles)")
+                return
+        self.linear(x, weight, out, tiles)
+        ops.call("activation", out, out, name)
+
     @staticmethod
     def gated_linear_norm_takes(rows: int, dtype, in_features: int) -> bool:
         """The gated product with the norm folded into its load of x: bfloat16, at most 16 rows,

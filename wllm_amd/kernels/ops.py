@@ -364,7 +364,7 @@ def head_prepare(rows: torch.Tensor, bias: Optional[torch.Tensor], positions: to
                  num_heads: int, num_kv_heads: int, head_dim: int, page_size: int, interleaved: bool = False,
                  norm_eps: Optional[float] = None, values_are_keys: bool = False,
                  parts: Optional[torch.Tensor] = None, norm_dim: Optional[int] = None,
-                 head_norm: Optional[tuple] = None, rot_scale: float = 1.0) -> None:
+                 head_norm: Optional[tuple] = None, rot_scale: float = 1.0, q_temperature: Optional[tuple] = None) -> None:
     """What `rope_and_cache_write` does, for attention blocks that do more between projection and
     attention.  rows T [n, width]: num_heads query heads, num_kv_heads key heads, num_kv_heads value
     heads unless `values_are_keys`, then any further columns.  In this order, in float32: every
@@ -379,7 +379,9 @@ def head_prepare(rows: torch.Tensor, bias: Optional[torch.Tensor], positions: to
     key heads stored.  slots, cache as in `rope_and_cache_write` (both None: nothing is stored).
     `head_norm` = (w_q, w_k, eps), float32 [head_dim] each: before the rotation every query head is divided by
     sqrt(sum of its squares / norm_dim + eps) and multiplied by w_q, every key head likewise by w_k (an RMS
-    norm with a weight over each head).  `rot_scale`: sine and cosine are multiplied by it."""
+    norm with a weight over each head).  `rot_scale`: sine and cosine are multiplied by it.
+    `q_temperature` = (coef, every): behind the norm every query head is multiplied by
+    1 + coef * ln(floor((position + 1) / every) + 1), in float32."""
     heads = num_heads + (1 if values_are_keys else 2) * num_kv_heads
     _dense(rows, "rows", _ACT)
     _need(rows.dim() == 2 and rows.shape[1] >= heads * head_dim,
@@ -415,6 +417,10 @@ def head_prepare(rows: torch.Tensor, bias: Optional[torch.Tensor], positions: to
         extra["head_norm"] = (w_q, w_k, float(pre_eps))
     if rot_scale != 1.0:
         extra["rot_scale"] = float(rot_scale)
+    if q_temperature is not None:
+        coef, every = q_temperature
+        _need(isinstance(every, int) and every > 0, "q_temperature: a coefficient and a positive number of positions")
+        extra["q_temperature"] = (float(coef), every)
     if n:
         call("head_prepare", rows, bias, positions, inv_freq, slots, cache, num_heads, num_kv_heads, head_dim,
              page_size, bool(interleaved), norm_eps, bool(values_are_keys), parts, norm_dim, **extra)
@@ -629,6 +635,39 @@ def gated_activation(gate_up: torch.Tensor, out: torch.Tensor, activation) -> No
         call("gated_activation", gate_up, out, activation)
 
 
+# the activations of a feed-forward without a gate (`common.h` holds the same table)
+SINGLE_ACTIVATIONS = {**ACTIVATIONS, "squared_relu": len(ACTIVATIONS)}
+
+
+def activation(x: torch.Tensor, out: torch.Tensor, name: str) -> None:
+    """out = act(x) in float32, cast to T; x, out T of one shape; out may be x."""
+    _need(name in SINGLE_ACTIVATIONS, lambda: f"activation {name!r}: expected one of {sorted(SINGLE_ACTIVATIONS)}")
+    _dense(x, "x", _ACT)
+    _dense(out, "out", x.dtype, tuple(x.shape))
+    if x.numel():
+        call("activation", x, out, name)
+
+
+def activated_linear(x: torch.Tensor, weight: torch.Tensor, out: torch.Tensor, name: str,
+                     tiles: Optional[torch.Tensor] = None, paired_tiles: Optional[torch.Tensor] = None) -> None:
+    """out = act(x @ weight^T).  x T [m, k]; weight T [n, k]; out T [m, n]; `tiles`: `tile_weight(weight)`; `paired_tiles`:
+    `tile_weight(weight, halves=2)` (n even), which the kernels that apply the activation in their registers read.  Where the
+    product and the activation are two kernels the product is rounded to T between them."""
+    _need(name in SINGLE_ACTIVATIONS, lambda: f"activation {name!r}: expected one of {sorted(SINGLE_ACTIVATIONS)}")
+    _dense(x, "x", _ACT)
+    _need(x.dim() == 2, "x: expected [rows, in]")
+    _dense(weight, "weight", x.dtype)
+    _need(weight.dim() == 2 and weight.shape[1] == x.shape[1],
+          lambda: f"weight: shape {tuple(weight.shape)}, expected [out, {x.shape[1]}]")
+    _dense(out, "out", x.dtype, (x.shape[0], weight.shape[0]))
+    _check_tiles(tiles, weight, 1)
+    if paired_tiles is not None:
+        _need(weight.shape[0] % 2 == 0, "paired_tiles: an even number of columns")
+        _check_tiles(paired_tiles, weight, 2)
+    if x.shape[0]:
+        backend().activated_linear(x, weight, out, name, tiles, paired_tiles)
+
+
 class NormOnLoad:
     """The input of a product as something the product kernel computes while it reads it:
     rms_norm(residual) with the rows' sums of squares already known.  residual float32 [m, k];
@@ -757,8 +796,13 @@ class NormRecipe:
 
 def norm_add(x: torch.Tensor, *, delta: Optional[torch.Tensor] = None, delta_norm: Optional[NormRecipe] = None,
              out: Optional[torch.Tensor] = None, out_norm: Optional[NormRecipe] = None,
-             rows: Optional[torch.Tensor] = None, conv: Optional[tuple] = None) -> None:
+             rows: Optional[torch.Tensor] = None, conv: Optional[tuple] = None, x_scale: float = 1.0,
+             sum_norm: Optional[NormRecipe] = None, extra: Optional[torch.Tensor] = None,
+             extra_scale: Optional[torch.Tensor] = None) -> None:
     """x += delta_norm(delta); out = out_norm(x), all in float32.
+    In general x = sum_norm(x_scale * x + delta_norm(delta + extra_scale * extra)): the stream may be weighed before the
+    sum, the sum may pass a norm of its own, and delta may have a second term, `extra` (T [n, H] or a stack float32
+    [S, n, H]), whose row i is multiplied by extra_scale[i] (float32 [n]; None: 1).
 
     x float32 [n, H], the residual stream.  delta T [n, H] or a stack float32 [S, n, H] of partial sums
     added in order; with `delta_norm` it is normalised before it is added (a norm behind a sublayer).
@@ -779,8 +823,8 @@ def norm_add(x: torch.Tensor, *, delta: Optional[torch.Tensor] = None, delta_nor
         else:
             _dense(delta, "delta", _ACT, (n, h))
     else:
-        _need(delta_norm is None, "delta_norm without delta")
-    for recipe, name in ((delta_norm, "delta_norm"), (out_norm, "out_norm")):
+        _need(delta_norm is None and sum_norm is None and extra is None and x_scale == 1.0, "delta_norm, sum_norm, extra, x_scale: with a delta")
+    for recipe, name in ((delta_norm, "delta_norm"), (out_norm, "out_norm"), (sum_norm, "sum_norm")):
         if recipe is not None:
             _need(tuple(recipe.weight.shape) == (h,), lambda: f"{name}: weight of {tuple(recipe.weight.shape)}, expected [{h}]")
     m = n
@@ -793,7 +837,23 @@ def norm_add(x: torch.Tensor, *, delta: Optional[torch.Tensor] = None, delta_nor
         _dense(out, "out", _ACT, (m, h))
     else:
         _need(out_norm is None, "out_norm without out")
-    extra = {}
+    _need(math.isfinite(x_scale), "x_scale: a finite number")
+    options = {}
+    if x_scale != 1.0:
+        options["x_scale"] = float(x_scale)
+    if sum_norm is not None:
+        options["sum_norm"] = sum_norm
+    if extra is not None:
+        if extra.dim() == 3:
+            _dense(extra, "extra", torch.float32, (extra.shape[0], n, h))
+            _need(extra.shape[0] >= 1, "extra: an empty stack")
+        else:
+            _dense(extra, "extra", _ACT, (n, h))
+        options["extra"] = extra
+    if extra_scale is not None:
+        _need(extra is not None, "extra_scale without extra")
+        _dense(extra_scale, "extra_scale", torch.float32, (n,))
+        options["extra_scale"] = extra_scale
     if conv is not None:
         weight, state, carried_offset, state_slots = conv
         _need(out is not None and out_norm is None and rows is None, "conv: with out, without out_norm and rows")
@@ -803,9 +863,9 @@ def norm_add(x: torch.Tensor, *, delta: Optional[torch.Tensor] = None, delta_nor
         _need(state.dim() == 2 and 0 <= carried_offset and carried_offset + (weight.shape[0] - 1) * h <= state.shape[1],
               "conv state: a row holds the carried rows from carried_offset")
         _dense(state_slots, "conv state_slots", torch.int32, (n,))
-        extra["conv"] = (weight, state, int(carried_offset), state_slots)
+        options["conv"] = (weight, state, int(carried_offset), state_slots)
     if m and (delta is not None or out is not None):
-        call("norm_add", x, delta, delta_norm, out, out_norm, rows, **extra)
+        call("norm_add", x, delta, delta_norm, out, out_norm, rows, **options)
 
 
 def band_norm(bands: list, eps: float) -> None:
@@ -1116,6 +1176,95 @@ def head_norm_gate(y: torch.Tensor, gate: Optional[torch.Tensor], weight: Option
         call("head_norm_gate", y, gate, weight, out, heads, float(eps), activation, float(scale), nq, floor, float(den_eps))
 
 
+# ---- a delta rule with a decay a key channel -------------------------------------------------------------
+DELTA_MAX_DIM = 256
+
+
+def delta_padded(dim: int) -> int:
+    """The channels of a head as the recurrence's operands and the memory hold them: a multiple of four."""
+    return -(-dim // 4) * 4
+
+
+def delta_state_size(heads: int, head_dim: int, value_dim: int) -> int:
+    """Floats of a request's memory: [heads, value_dim, delta_padded(head_dim)]."""
+    return heads * value_dim * delta_padded(head_dim)
+
+
+def _delta_sizes(heads: int, groups: int, head_dim: int, value_dim: int) -> None:
+    _need(heads > 0 and groups > 0 and heads % groups == 0, "heads must be a multiple of groups")
+    _need(0 < head_dim <= DELTA_MAX_DIM and value_dim > 0, f"head_dim: from 1 to {DELTA_MAX_DIM}")
+
+
+def delta_inputs(xqkv: torch.Tensor, z: torch.Tensor, b: torch.Tensor, conv_weight: torch.Tensor, rate: torch.Tensor,
+                 dt_bias: torch.Tensor, state: torch.Tensor, carried_offset: int, token_segment: torch.Tensor,
+                 seg_q_start: torch.Tensor, seg_q_len: torch.Tensor, state_slots: torch.Tensor, qk: torch.Tensor,
+                 kq: torch.Tensor, v: torch.Tensor, f: torch.Tensor, beta: torch.Tensor, *, heads: int, groups: int,
+                 head_dim: int, value_dim: int, q_scale: float, unit_eps: float, single_tokens: bool = False) -> None:
+    """A gated delta rule's operands from a token's projections, in float32:
+        [q | k | v] = silu(short causal convolution of xqkv);  q, k = unit vectors a head, x / sqrt(sum(x^2) + unit_eps),
+        q times q_scale;  f = exp(-rate softplus(z + dt_bias));  beta = sigmoid(b);  kq = k . q
+    xqkv T [n, 2 * groups * D + heads * P] (D = head_dim, P = value_dim), z T [n, heads * D] and b T [n, heads] may be bands of
+    wider rows; conv_weight float32 [taps, channels], a row a tap, the last the current token's; rate float32 [heads];
+    dt_bias float32 [heads * D].  Inputs before a segment's first token are the request's carried rows: state float32
+    [slots, W] holds [taps - 1, channels], the oldest first, from column `carried_offset` of row state_slots[segment]
+    (zeros for a fresh request); afterwards they are the segment's last taps - 1 inputs.  With DP = delta_padded(D): qk
+    float32 [2, n, groups * DP] and f float32 [n, heads * DP] (zeros in the padding), kq float32 [n, groups], v T
+    [n, heads * P], beta float32 [n, heads].  `single_tokens`: every segment is one token (a decode step), and the launch
+    that reads the carried rows moves them."""
+    _delta_sizes(heads, groups, head_dim, value_dim)
+    _need(xqkv.dim() == 2 and xqkv.dtype in _ACT, "xqkv: expected T [n, channels]")
+    n, channels, dp = xqkv.shape[0], 2 * groups * head_dim + heads * value_dim, delta_padded(head_dim)
+    _band(xqkv, "xqkv", xqkv.dtype, n, channels)
+    _band(z, "z", xqkv.dtype, n, heads * head_dim)
+    _band(b, "b", xqkv.dtype, n, heads)
+    _dense(conv_weight, "conv_weight", torch.float32)
+    _need(conv_weight.dim() == 2 and conv_weight.shape[1] == channels and 1 <= conv_weight.shape[0] <= 64,
+          lambda: f"conv_weight: expected [taps <= 64, {channels}]")
+    _dense(rate, "rate", torch.float32, (heads,))
+    _dense(dt_bias, "dt_bias", torch.float32, (heads * head_dim,))
+    _dense(state, "state", torch.float32)
+    _need(state.dim() == 2 and 0 <= carried_offset and carried_offset + (conv_weight.shape[0] - 1) * channels <= state.shape[1],
+          "state: a row holds the carried rows from carried_offset")
+    _dense(token_segment, "token_segment", torch.int32, (n,))
+    s = _segments(seg_q_start, seg_q_len, state_slots)
+    _need(not single_tokens or s == n, "single_tokens: as many segments as tokens")
+    _dense(qk, "qk", torch.float32, (2, n, groups * dp))
+    _dense(kq, "kq", torch.float32, (n, groups))
+    _dense(v, "v", xqkv.dtype, (n, heads * value_dim))
+    _dense(f, "f", torch.float32, (n, heads * dp))
+    _dense(beta, "beta", torch.float32, (n, heads))
+    if n:
+        call("delta_inputs", xqkv, z, b, conv_weight, rate, dt_bias, state, int(carried_offset), token_segment, seg_q_start,
+             seg_q_len, state_slots, qk, kq, v, f, beta, heads, groups, head_dim, value_dim, float(q_scale), float(unit_eps),
+             bool(single_tokens))
+
+
+def delta_scan(qk: torch.Tensor, kq: torch.Tensor, f: torch.Tensor, beta: torch.Tensor, v: torch.Tensor, state: torch.Tensor,
+               seg_q_start: torch.Tensor, seg_q_len: torch.Tensor, state_slots: torch.Tensor, y: torch.Tensor, *, heads: int,
+               groups: int, head_dim: int, value_dim: int) -> None:
+    """The delta rule over each segment's tokens in order, from and into the request's carried memory.  Per head h (group
+    h // (heads // groups) of q and k):  S = diag(f) S;  u = beta (v - S^T k);  S += k u^T;  y = S^T q, the last computed as
+    (diag(f) S)^T q + u (k . q).  Operands as `delta_inputs` leaves them; state float32 [slots, W] (W a multiple of four),
+    whose row state_slots[segment] begins with [heads, P, DP]: a head's memory, a value column after the other;
+    y float32 [n, heads * P].  All float32."""
+    _delta_sizes(heads, groups, head_dim, value_dim)
+    dp = delta_padded(head_dim)
+    _need(v.dim() == 2 and v.dtype in _ACT, "v: expected T [n, heads * value_dim]")
+    n = v.shape[0]
+    _dense(v, "v", _ACT, (n, heads * value_dim))
+    _dense(qk, "qk", torch.float32, (2, n, groups * dp))
+    _dense(kq, "kq", torch.float32, (n, groups))
+    _dense(f, "f", torch.float32, (n, heads * dp))
+    _dense(beta, "beta", torch.float32, (n, heads))
+    _dense(state, "state", torch.float32)
+    _need(state.dim() == 2 and state.shape[1] >= delta_state_size(heads, head_dim, value_dim) and state.shape[1] % 4 == 0,
+          "state: a row begins with [heads, P, DP] and is a multiple of four floats")
+    _segments(seg_q_start, seg_q_len, state_slots)
+    _dense(y, "y", torch.float32, (n, heads * value_dim))
+    if n:
+        call("delta_scan", qk, kq, f, beta, v, state, seg_q_start, seg_q_len, state_slots, y, heads, groups, head_dim, value_dim)
+
+
 # ---- a mixture of experts ------------------------------------------------------------------------------
 MOE_TILE_ROWS = 16           # rows of a tile of the kernels that stream an expert's weights past a few rows: 16, 32 or 64
 MOE_STREAM_TILE_ROWS = (16, 32, 64)
@@ -1151,21 +1300,25 @@ MOE_SCORINGS = {"softmax": 0, "sigmoid": 1}
 
 
 def moe_route(x: torch.Tensor, router: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor, *, groups: int = 1,
-              keep: int = 1, eps: float = 1e-20, scoring: str = "softmax", normalize: bool = True) -> None:
+              keep: int = 1, eps: float = 1e-20, scoring: str = "softmax", normalize: bool = True,
+              correction: Optional[torch.Tensor] = None, group_best: int = 1, gates: Optional[torch.Tensor] = None) -> None:
     """Which experts each token uses.  z = x router^T in float32; s = softmax(z) over all experts; the
     experts form `groups` equal groups of neighbours, a group's score is its largest s, and only experts of
     the `keep` best groups may be chosen; the `top` = ids.shape[1] allowed experts with the largest s are
     chosen (of equal scores the lower index first), weights = their s / (sum of the chosen + eps).
     `scoring` "sigmoid": s = sigmoid(z), every expert by itself.  `normalize` False: weights = the chosen s themselves.
+    `correction` (float32 [experts]): what decides every choice is c = s + correction (which may be negative); the weights
+    come of s alone.  `group_best` 2: a group's score is the sum of its two largest c (of its only one, if it has one).
+    `gates` (float32 [n]): router has one more row behind the experts', and gates takes the sigmoid of its product.
     x T [n, width]; router float32 [experts, width]; ids int32 [n, top]; weights float32 [n, top]."""
     _need(scoring in MOE_SCORINGS, lambda: f"scoring {scoring!r}: one of {sorted(MOE_SCORINGS)}")
     _dense(x, "x", _ACT)
     _need(x.dim() == 2, "x: expected [n, width]")
     n, width = x.shape
     _dense(router, "router", torch.float32)
-    _need(router.dim() == 2 and router.shape[1] == width and 0 < router.shape[0] <= MOE_MAX_EXPERTS,
+    experts = router.shape[0] - (1 if gates is not None else 0)
+    _need(router.dim() == 2 and router.shape[1] == width and 0 < experts <= MOE_MAX_EXPERTS,
           lambda: f"router: expected [at most {MOE_MAX_EXPERTS} experts, {width}]")
-    experts = router.shape[0]
     _dense(ids, "ids", torch.int32)
     _need(ids.dim() == 2 and ids.shape[0] == n, "ids: expected [n, top]")
     top = ids.shape[1]
@@ -1174,6 +1327,15 @@ def moe_route(x: torch.Tensor, router: torch.Tensor, ids: torch.Tensor, weights:
     _need(0 < top <= keep * (experts // groups), "top: at most the experts of the kept groups")
     if n:
         extra = {} if scoring == "softmax" and normalize else {"scoring": scoring, "normalize": bool(normalize)}
+        if correction is not None:
+            _dense(correction, "correction", torch.float32, (experts,))
+            extra["correction"] = correction
+        _need(group_best in (1, 2), "group_best: 1 or 2")
+        if group_best != 1:
+            extra["group_best"] = group_best
+        if gates is not None:
+            _dense(gates, "gates", torch.float32, (n,))
+            extra["gates"] = gates
         call("moe_route", x, router, ids, weights, int(groups), int(keep), float(eps), **extra)
 
 
@@ -1283,8 +1445,13 @@ def _register_own() -> None:
                     out.shape[1], out.stride(0) if out.shape[0] > 1 else out.shape[1], stream))
 
 
+    register_op("activation", entry_point="wllm_activation", argtypes=[c_void_p, c_void_p, c_int, c_int, c_longlong, c_void_p],
+                launch=lambda fn, stream, x, out, name: fn(
+                    p(x), p(out), int(x.dtype == torch.bfloat16), SINGLE_ACTIVATIONS[name], x.numel(), stream))
+
     def prepare(fn, stream, rows, bias, positions, inv_freq, slots, cache, num_heads, num_kv_heads, head_dim,
-                page_size, interleaved, norm_eps, values_are_keys, parts, norm_dim, head_norm=None, rot_scale=1.0):
+                page_size, interleaved, norm_eps, values_are_keys, parts, norm_dim, head_norm=None, rot_scale=1.0,
+                q_temperature=(0.0, 0)):
         w_q, w_k, pre_eps = head_norm if head_norm is not None else (None, None, -1.0)
         splits, stride = (parts.shape[0], parts.shape[1] * parts.shape[2]) if parts is not None else (0, 0)
         return fn(p(rows), int(rows.dtype == torch.bfloat16), rows.shape[1], p(parts), splits, stride, p(bias),
@@ -1292,12 +1459,12 @@ def _register_own() -> None:
                   rows.shape[0], num_heads, num_kv_heads, head_dim,
                   2 * inv_freq.shape[0] if inv_freq is not None else 0, int(interleaved),
                   float(norm_eps) if norm_eps is not None else -1.0, norm_dim, int(values_are_keys), page_size,
-                  p(w_q), p(w_k), pre_eps, rot_scale, stream)
+                  p(w_q), p(w_k), pre_eps, rot_scale, *q_temperature, stream)
 
     register_op("head_prepare", entry_point="wllm_head_prepare",
                 argtypes=[c_void_p, c_int, c_int, c_void_p, c_int, c_longlong, c_void_p, c_int, c_void_p, c_void_p, c_void_p,
                           c_void_p, c_longlong, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_int, c_int, c_void_p,
-                          c_void_p, c_float, c_float, c_void_p],
+                          c_void_p, c_float, c_float, c_float, c_int, c_void_p],
                 launch=prepare)
     register_op("sigmoid_gate", entry_point="wllm_sigmoid_gate",
                 argtypes=[c_void_p, c_longlong, c_void_p, c_longlong, c_void_p, c_longlong, c_int, c_int, c_int, c_int,
@@ -1323,8 +1490,11 @@ def _register_own() -> None:
                 launch=add)
 
 
-    def norm_add_launch(fn, stream, x, delta, delta_norm, out, out_norm, rows, conv=None):
-        splits, stride = 1, 0
+    def norm_add_launch(fn, stream, x, delta, delta_norm, out, out_norm, rows, conv=None, x_scale=1.0, sum_norm=None,
+                        extra=None, extra_scale=None):
+        splits, stride, extra_splits, extra_stride = 1, 0, 1, 0
+        if extra is not None and extra.dim() == 3:
+            extra_splits, extra_stride = extra.shape[0], extra.shape[1] * extra.shape[2]
         if delta is not None and delta.dim() == 3:
             splits, stride = delta.shape[0], delta.shape[1] * delta.shape[2]
 
@@ -1335,12 +1505,15 @@ def _register_own() -> None:
                   *recipe(delta_norm), p(rows), p(out), int(out is not None and out.dtype == torch.bfloat16),
                   *recipe(out_norm), out.shape[0] if out is not None else x.shape[0], x.shape[1],
                   *((p(conv[0]), conv[0].shape[0], p(conv[1]), conv[1].stride(0), conv[2], p(conv[3])) if conv is not None
-                    else (p(None), 0, p(None), 0, 0, p(None))), stream)
+                    else (p(None), 0, p(None), 0, 0, p(None))),
+                  x_scale, *recipe(sum_norm), p(extra), int(extra is not None and extra.dtype == torch.bfloat16), extra_splits,
+                  extra_stride, p(extra_scale), stream)
 
     register_op("norm_add", entry_point="wllm_norm_add",
                 argtypes=[c_void_p, c_void_p, c_int, c_int, c_longlong, c_int, c_void_p, c_float, c_float, c_void_p, c_void_p,
                           c_int, c_int, c_void_p, c_float, c_float, c_int, c_int, c_void_p, c_int, c_void_p, c_longlong,
-                          c_longlong, c_void_p, c_void_p],
+                          c_longlong, c_void_p, c_float, c_int, c_void_p, c_float, c_float, c_void_p, c_int, c_int, c_longlong,
+                          c_void_p, c_void_p],
                 launch=norm_add_launch)
 
     def band_norm_launch(fn, stream, bands, eps):
@@ -1431,12 +1604,29 @@ def _register_own() -> None:
                 den_eps=0.0: fn(
                     p(y), p(gate), gate.stride(0) if gate is not None else 0, p(weight), p(out), out.stride(0), p(nq), p(floor),
                     den_eps, bf(out), GATE_KINDS[activation], y.shape[0], heads, y.shape[1] // heads, eps, scale, stream))
+    register_op("delta_inputs", entry_point="wllm_delta_inputs",
+                argtypes=[c_void_p, c_longlong, c_void_p, c_longlong, c_void_p, c_longlong, c_void_p, c_void_p, c_void_p, c_void_p,
+                          c_longlong, c_longlong] + [c_void_p] * 9 + [c_float, c_float] + [c_int] * 9 + [c_void_p],
+                launch=lambda fn, stream, xqkv, z, b, conv_weight, rate, dt_bias, state, carried_offset, token_segment, seg_q_start,
+                seg_q_len, state_slots, qk, kq, v, f, beta, heads, groups, head_dim, value_dim, q_scale, unit_eps, single_tokens: fn(
+                    p(xqkv), xqkv.stride(0), p(z), z.stride(0), p(b), b.stride(0), p(conv_weight), p(rate), p(dt_bias), p(state),
+                    state.stride(0), carried_offset, p(token_segment), p(seg_q_start), p(seg_q_len), p(state_slots), p(qk), p(kq),
+                    p(v), p(f), p(beta), q_scale, unit_eps, bf(xqkv), xqkv.shape[0], seg_q_start.shape[0], heads, groups, head_dim,
+                    value_dim, conv_weight.shape[0], int(single_tokens), stream))
+    register_op("delta_scan", entry_point="wllm_delta_scan",
+                argtypes=[c_void_p] * 6 + [c_longlong] + [c_void_p] * 4 + [c_int] * 7 + [c_void_p],
+                launch=lambda fn, stream, qk, kq, f, beta, v, state, seg_q_start, seg_q_len, state_slots, y, heads, groups, head_dim,
+                value_dim: fn(
+                    p(qk), p(kq), p(f), p(beta), p(v), p(state), state.stride(0), p(seg_q_start), p(seg_q_len), p(state_slots), p(y),
+                    bf(v), v.shape[0], seg_q_start.shape[0], heads, groups, head_dim, value_dim, stream))
     register_op("moe_route", entry_point="wllm_moe_route",
-                argtypes=[c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float,
-                          c_int, c_int, c_void_p],
-                launch=lambda fn, stream, x, router, ids, weights, groups, keep, eps, scoring="softmax", normalize=True: fn(
-                    p(x), p(router), p(ids), p(weights), bf(x), x.shape[0], x.shape[1], router.shape[0], ids.shape[1], groups,
-                    keep, eps, MOE_SCORINGS[scoring], int(normalize), stream))
+                argtypes=[c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int,
+                          c_int, c_int, c_float, c_int, c_int, c_void_p],
+                launch=lambda fn, stream, x, router, ids, weights, groups, keep, eps, scoring="softmax", normalize=True,
+                correction=None, group_best=1, gates=None: fn(
+                    p(x), p(router), p(correction), p(ids), p(weights), p(gates), bf(x), x.shape[0], x.shape[1],
+                    router.shape[0] - (1 if gates is not None else 0), ids.shape[1], groups, keep, group_best, eps,
+                    MOE_SCORINGS[scoring], int(normalize), stream))
     register_op("moe_plan", entry_point="wllm_moe_plan", argtypes=[c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_void_p],
                 launch=lambda fn, stream, ids, plan, experts, tile_rows=MOE_TILE_ROWS: fn(
                     p(ids), p(plan), ids.numel(), experts, moe_max_tiles(ids.numel(), experts, tile_rows), tile_rows, stream))

@@ -20,7 +20,7 @@ the row and in the cache, with zeros that add nothing to a score or a result); a
 instead of a window; an RMS norm with a weight over the whole query projection and over the whole key
 projection (`ops.band_norm`) in place of the norm of each head; a gate of one number a head; and a
 layer without key and value projections that reads another layer's cache with its own queries.
-And: an RMS norm with a weight over every query head and every key head before the rotation (the weight
+And: a temperature on the queries that grows with the position (behind the unit norm); an RMS norm with a weight over every query head and every key head before the rotation (the weight
 has head_dim numbers that the heads share), and a learned number a head in the softmax's denominator.
 """
 from __future__ import annotations
@@ -50,7 +50,8 @@ class PagedAttention:
                      or spec.position.pairing == "interleaved" or spec.value_dim not in (None, spec.head_dim)
                      or spec.chunk or spec.q_norm_weight or spec.k_norm_weight or not spec.owns_cache
                      or spec.sink is not None or spec.output_scale != 1.0 or spec.q_head_norm_weight
-                     or spec.k_head_norm_weight or spec.sink_weight or spec.position.magnitude != 1.0)
+                     or spec.k_head_norm_weight or spec.sink_weight or spec.position.magnitude != 1.0
+                     or spec.q_temperature is not None)
         if bool(spec.q_head_norm_weight) != bool(spec.k_head_norm_weight) or (
                 spec.q_head_norm_weight and (spec.head_norm_eps is None or spec.head_norm_eps < 0)):
             raise ValueError("a norm over each head has a weight for the queries, one for the keys, and head_norm_eps")
@@ -58,6 +59,9 @@ class PagedAttention:
             raise ValueError("a norm over each head and a norm over the whole projection: one of the two")
         if spec.q_head_norm_weight and not spec.owns_cache:
             raise ValueError("a norm over each head: the layer has keys of its own")
+        if spec.q_temperature is not None and (not spec.owns_cache or not isinstance(spec.q_temperature[1], int)
+                                               or spec.q_temperature[1] <= 0):
+            raise ValueError("q_temperature: a coefficient and a positive number of positions, on a layer with keys of its own")
         if spec.sink_weight and spec.sink is not None:
             raise ValueError("sink and sink_weight: the denominator's term is a constant or a learned number a head")
         if spec.chunk is not None and (spec.chunk <= 0 or spec.window is not None):
@@ -287,7 +291,8 @@ class PagedAttention:
                     qkv, self.b_qkv, ctx.positions, inv_freq, slots, storage, num_heads=s.num_heads,
                     num_kv_heads=s.num_kv_heads, head_dim=self.dim, page_size=pages.page_size,
                     interleaved=getattr(self.position, "interleaved", False), norm_eps=s.qk_norm_eps,
-                    values_are_keys=s.values_are_keys, norm_dim=s.head_dim, rot_scale=getattr(self.position, "magnitude", 1.0))
+                    values_are_keys=s.values_are_keys, norm_dim=s.head_dim, rot_scale=getattr(self.position, "magnitude", 1.0),
+                    q_temperature=s.q_temperature)
         elif not self.plain:
             if apply is not None:
                 raise NotImplementedError("a position encoding with a step of its own beside the attention's options")
@@ -298,7 +303,8 @@ class PagedAttention:
                 interleaved=getattr(self.position, "interleaved", False), norm_eps=s.qk_norm_eps,
                 values_are_keys=s.values_are_keys, parts=projected if projected.dim() == 3 else None,
                 norm_dim=s.head_dim, rot_scale=getattr(self.position, "magnitude", 1.0),
-                head_norm=(self.w_q_head_norm, self.w_k_head_norm, s.head_norm_eps) if self.w_q_head_norm is not None else None)
+                head_norm=(self.w_q_head_norm, self.w_k_head_norm, s.head_norm_eps) if self.w_q_head_norm is not None else None,
+                q_temperature=s.q_temperature)
         elif apply is not None:
             ops.linear(h, self.w_qkv, qkv, self.t_qkv)
             if self.b_qkv is not None:

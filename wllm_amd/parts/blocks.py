@@ -24,6 +24,9 @@ the stream itself, optionally through a short convolution over time (`InputConv`
 a weighted sum of its last few values, channel by channel).  The convolution's last inputs are state that
 the block, not its mixer, carries for a request: the block names it in `state_shapes()` and finds it
 under (run, name).
+
+"norm_of_sum": x = post(w x + mixer(x)); x = post(w x + feed_forward(x)): as "post_norm", but the norm behind a
+sublayer takes the sum of the weighed stream and the sublayer's result, and what it gives is the stream.
 """
 from __future__ import annotations
 
@@ -32,7 +35,7 @@ from typing import Optional
 import torch
 
 from wllm_amd.kernels import ops
-from wllm_amd.parts.common import Product
+from wllm_amd.parts.common import Product, TwoTerms
 from wllm_amd.parts.registry import build_feed_forward, build_mixer, build_norm, register_block
 from wllm_amd.parts.specs import BlockSpec, InputConvSpec
 from wllm_amd.weights.checkpoint import ExpectedTensor
@@ -53,16 +56,36 @@ class ResidualStream:
         self.pending = pending
         self.pending_bias: Optional[torch.Tensor] = None      # float32 [H]: a row that comes with `pending`
         self.pending_norm = None       # an `ops.NormRecipe`: `pending` passes this norm before it is added
+        self.pending_extra = None      # (tensor, scale or None): a second term of what is pending
+        self.pending_sum = None        # (weight of x, `ops.NormRecipe`): the sum passes this norm and is the new x
         self.sumsq: Optional[torch.Tensor] = None      # float32 [n, bands]: sums of squares of x as it is now
+
+    @property
+    def joins(self) -> bool:
+        """Whether what is pending is more than an addend: only `ops.norm_add` brings it in."""
+        return self.pending_norm is not None or self.pending_extra is not None or self.pending_sum is not None
+
+    def join_options(self) -> dict:
+        """What is pending, as `ops.norm_add` takes it."""
+        options = {"delta": self.pending, "delta_norm": self.pending_norm}
+        if self.pending_extra is not None:
+            options["extra"], options["extra_scale"] = self.pending_extra
+        if self.pending_sum is not None:
+            options["x_scale"], options["sum_norm"] = self.pending_sum
+        return options
+
+    def joined(self) -> None:
+        """What was pending is in x."""
+        self.pending = self.pending_norm = self.pending_extra = self.pending_sum = None
+        self.sumsq = None
 
     def normed(self, norm, out: torch.Tensor, rows=None) -> torch.Tensor:
         """norm(x + pending).  Without `rows` the sum becomes the new x."""
-        if self.pending_norm is not None:
+        if self.joins:
             if getattr(norm, "takes_delta_norm", False) and self.pending_bias is None:
-                norm.forward(self.x, out, delta=self.pending, rows=rows, delta_norm=self.pending_norm)
+                ops.norm_add(self.x, out=out, out_norm=norm.recipe(), rows=rows, **self.join_options())
                 if rows is None:
-                    self.pending = self.pending_norm = None
-                    self.sumsq = None
+                    self.joined()
                 return out
             if rows is not None:
                 raise NotImplementedError("gathered rows of a stream whose pending part has a norm, under a norm "
@@ -81,10 +104,9 @@ class ResidualStream:
         """x takes what is pending, and `addend` (float32, x's shape) with it, without a norm."""
         if self.pending is None and self.pending_bias is None and addend is None:
             return
-        if self.pending_norm is not None:
-            ops.norm_add(self.x, delta=self.pending, delta_norm=self.pending_norm)
-            self.pending = self.pending_norm = None
-            self.sumsq = None
+        if self.joins:
+            ops.norm_add(self.x, **self.join_options())
+            self.joined()
             if self.pending_bias is None and addend is None:
                 return
         ops.stream_add(self.x, addend, self.pending, self.pending_bias)
@@ -110,21 +132,29 @@ class ResidualStream:
         out = ctx.buffer("stream_cast", (n, hidden), ctx.dtype)
         if self.pending_bias is not None:
             self.settle()
-        ops.norm_add(self.x, delta=self.pending, delta_norm=self.pending_norm, out=out)
-        self.pending = self.pending_norm = None
-        self.sumsq = None
+        ops.norm_add(self.x, out=out, **self.join_options())
+        self.joined()
         return out
 
-    def add(self, ctx, y, norm=None) -> None:
-        """`norm` (a norm part): the contribution passes it before it is added (a norm behind a sublayer)."""
+    def add(self, ctx, y, norm=None, sum_norm=None, weight: float = 1.0) -> None:
+        """`norm` (a norm part): the contribution passes it before it is added (a norm behind a sublayer).  `sum_norm`:
+        the sum of `weight` times the stream and the contribution passes it instead and becomes the stream."""
         if self.pending is not None or self.pending_bias is not None:
             raise RuntimeError("a contribution is already pending; normalise before adding another")
-        if norm is not None:
+        if isinstance(y, TwoTerms):
+            if y.extra.bias is not None:
+                raise NotImplementedError("a second term with a bias")
+            self.pending_extra = (y.extra.make(ctx), y.scale)
+            y = y.delta
+        elif norm is not None or sum_norm is not None:
             if isinstance(y, Product):
                 if y.bias is not None:
                     raise NotImplementedError("a product with a bias under a norm behind its sublayer")
                 y = y.make(ctx)
-            self.pending, self.pending_norm = y, norm.recipe()
+        if norm is not None or sum_norm is not None or self.pending_extra is not None:
+            self.pending = y
+            self.pending_norm = norm.recipe() if norm is not None else None
+            self.pending_sum = (weight, sum_norm.recipe()) if sum_norm is not None else None
             return
         if isinstance(y, Product):
             n, hidden = self.x.shape
@@ -284,10 +314,8 @@ class InputConv:
         single = ctx.max_q_len == 1 and ctx.num_segments == n       # a step of single tokens, a captured graph among them
         if single and stream.pending is not None and stream.pending_bias is None:
             # no token reads another's row: the launch that settles the stream also convolves and moves the carried rows
-            ops.norm_add(stream.x, delta=stream.pending, delta_norm=stream.pending_norm, out=out,
-                         conv=(self.weight, state, offset, ctx.state_slots))
-            stream.pending = stream.pending_norm = None
-            stream.sumsq = None
+            ops.norm_add(stream.x, out=out, conv=(self.weight, state, offset, ctx.state_slots), **stream.join_options())
+            stream.joined()
             return out
         stream.settle()         # the convolution reads other tokens' rows of the stream: they take what is pending first
         ops.stream_conv(stream.x, self.weight, state, offset, ctx.token_segment, ctx.seg_q_start, ctx.seg_q_len,
@@ -337,8 +365,19 @@ class PostNormBlock:
 
     def forward(self, ctx, entry: int, stream: ResidualStream) -> None:
         h = self._read(ctx, entry, stream, self.mixer_conv, 0)
-        stream.add(ctx, self.mixer.forward(ctx, entry, h), norm=self.mixer_post_norm)
+        self._add(ctx, stream, self.mixer.forward(ctx, entry, h), self.mixer_post_norm)
         if self.feed_forward is not None:
             offset = self.mixer_conv.carried if self.mixer_conv is not None else 0
             h = self._read(ctx, entry, stream, self.feed_forward_conv, offset)
-            stream.add(ctx, self.feed_forward.forward(ctx, h), norm=self.feed_forward_post_norm)
+            self._add(ctx, stream, self.feed_forward.forward(ctx, h), self.feed_forward_post_norm)
+
+    def _add(self, ctx, stream: ResidualStream, y, norm) -> None:
+        stream.add(ctx, y, norm=norm)
+
+
+@register_block("norm_of_sum")
+class NormOfSumBlock(PostNormBlock):
+    """x = post(w x + mixer(read(x))); x = post(w x + feed_forward(read(x))), read as in `PostNormBlock`."""
+
+    def _add(self, ctx, stream: ResidualStream, y, norm) -> None:
+        stream.add(ctx, y, sum_norm=norm, weight=self.spec.stream_weight)

@@ -41,6 +41,15 @@ class Product:
         return project(ctx, self.name, self.x, self.weight, tiles=self.tiles)
 
 
+class TwoTerms:
+    """A contribution to the residual stream in two terms, y = delta + scale * extra: `delta` a tensor or a float32 stack
+    of partial sums, `extra` a `Product`, `scale` float32 [rows] (a number a row) or None.  Whoever adds it forms the
+    sum in float32 (`ops.norm_add`)."""
+
+    def __init__(self, delta: torch.Tensor, extra: Product, scale: Optional[torch.Tensor] = None):
+        self.delta, self.extra, self.scale = delta, extra, scale
+
+
 def load_matrix(fetch, matrix: torch.Tensor, halves: int = 1):
     """A weight matrix on the device as the product kernels want it: (the matrix, row by row, for
     products of many rows; its tile-major copy for the few rows of a decode step, or None).  The

@@ -2,7 +2,7 @@
 with act = gelu_tanh it is the reference's GemmaMLP (src/wllm/models/gemma.py:54-62).
 "clamped_swish" holds the gate under a limit and the up projection between two, and raises the latter by a constant.
 Gate and up matrices are stacked at load so that one product makes both halves
-of the row the activation kernel reads."""
+of the row the activation kernel reads.  "mlp": down(act(up(x))), no gate."""
 from __future__ import annotations
 
 import torch
@@ -10,7 +10,7 @@ import torch
 from wllm_amd.kernels import ops
 from wllm_amd.parts.common import Product, load_matrix
 from wllm_amd.parts.registry import register_feed_forward
-from wllm_amd.parts.specs import GatedMLPSpec
+from wllm_amd.parts.specs import GatedMLPSpec, MLPSpec
 from wllm_amd.weights.checkpoint import ExpectedTensor
 
 
@@ -71,6 +71,43 @@ class GatedMLP:
                 act = ctx.buffer("ffn_act", (n, s.intermediate_size), h.dtype)
             ops.gated_linear(h, self.w_gate_up, act, self.activation, gate_up, self.t_gate_up)
         if product_input is not None and act is not product_input:
+            ops.copy_columns(act, product_input)
+            act = product_input
+        return Product("ffn_out", act, self.w_down, self.t_down)
+
+
+@register_feed_forward("mlp")
+class MLP:
+    """down(act(up(x))).  Where the few-row and tiled kernels of a gated product apply (bfloat16, an even number of
+    columns), the two halves of the columns are their two streams and the activation is made in their registers."""
+
+    def __init__(self, spec: MLPSpec):
+        if spec.activation not in ops.SINGLE_ACTIVATIONS:
+            raise ValueError(f"activation {spec.activation!r} is not implemented; known: {sorted(ops.SINGLE_ACTIVATIONS)}")
+        self.spec = spec
+        self.w_up = self.t_up = self.w_down = self.t_down = None
+        self.paired = False                 # t_up is tiled as two halves
+
+    def expected_tensors(self) -> dict:
+        s = self.spec
+        return {s.up_weight: ExpectedTensor((s.intermediate_size, s.hidden_size)),
+                s.down_weight: ExpectedTensor((s.hidden_size, s.intermediate_size))}
+
+    def load(self, fetch) -> None:
+        s = self.spec
+        self.paired = s.intermediate_size % 2 == 0 and fetch.dtype == torch.bfloat16
+        self.w_up, self.t_up = load_matrix(fetch, fetch.matrix(s.up_weight), halves=2 if self.paired else 1)
+        self.w_down, self.t_down = load_matrix(fetch, fetch.matrix(s.down_weight))
+
+    def flops(self, tokens: int) -> float:
+        return 4.0 * tokens * self.spec.hidden_size * self.spec.intermediate_size
+
+    def forward(self, ctx, h, product_input=None):
+        s = self.spec
+        act = ctx.buffer("ffn_act", (h.shape[0], s.intermediate_size), h.dtype)
+        ops.activated_linear(h, self.w_up, act, s.activation, None if self.paired else self.t_up,
+                             self.t_up if self.paired else None)
+        if product_input is not None:
             ops.copy_columns(act, product_input)
             act = product_input
         return Product("ffn_out", act, self.w_down, self.t_down)

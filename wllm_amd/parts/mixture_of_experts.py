@@ -19,7 +19,9 @@ Options: the scores may be sigmoids of the logits, every expert by itself (`scor
 may be the weights as they are (`normalize` False); the weight may multiply the expert's input instead of its
 output (`weight_on_input`: the factor is taken out of the first product's two sums and multiplied in before the
 activation, and the second product's results are not weighed); and one more gated feed-forward may run for
-every token (`shared`), whose result is one more slice of the stack.
+every token (`shared`), whose result is a second term that whoever adds the stack adds with it, multiplied by a sigmoid
+of its own if it has a gate (one more row of the router's product).  A correction may be added to the scores for the
+choices alone, and a group's score may be the sum of its two best.
 """
 from __future__ import annotations
 
@@ -27,6 +29,7 @@ import torch
 
 from wllm_amd.kernels import ops
 from wllm_amd.parts.feed_forward import GatedMLP
+from wllm_amd.parts.common import TwoTerms
 from wllm_amd.parts.registry import register_feed_forward
 from wllm_amd.parts.specs import MixtureOfExpertsSpec
 from wllm_amd.weights.checkpoint import ExpectedTensor
@@ -48,7 +51,12 @@ class MixtureOfExperts:
             raise ValueError(f"top ({spec.top}): at most the experts of the kept groups")
         if spec.scoring not in ops.MOE_SCORINGS:
             raise ValueError(f"scoring {spec.scoring!r}: one of {sorted(ops.MOE_SCORINGS)}")
+        if spec.group_best not in (1, 2):
+            raise ValueError(f"group_best {spec.group_best}: 1 or 2")
+        if spec.shared_gate_weight and spec.shared is None:
+            raise ValueError("shared_gate_weight without a shared expert")
         self.spec = spec
+        self.correction = None
         self.shared = GatedMLP(spec.shared) if spec.shared is not None else None
         self.w_router = self.w_up = self.w_down = None
         self.t_up = self.t_down = None          # the stacks' tile-major copies, which the few-row kernels stream
@@ -67,6 +75,10 @@ class MixtureOfExperts:
             out[gate] = ExpectedTensor((s.intermediate_size, s.hidden_size))
             out[up] = ExpectedTensor((s.intermediate_size, s.hidden_size))
             out[down] = ExpectedTensor((s.hidden_size, s.intermediate_size))
+        if s.correction_weight:
+            out[s.correction_weight] = ExpectedTensor((s.num_experts,), role="vector", init="norm")
+        if s.shared_gate_weight:
+            out[s.shared_gate_weight] = ExpectedTensor((1, s.hidden_size), role="vector")
         if self.shared is not None:
             out.update(self.shared.expected_tensors())
         return out
@@ -85,7 +97,11 @@ class MixtureOfExperts:
             downs.append(fetch.matrix(down))
         self.w_up = fetch.to_device(torch.stack(ups).contiguous())
         self.w_down = fetch.to_device(torch.stack(downs).contiguous())
-        self.w_router = fetch.to_device(fetch.vector(s.router_weight))
+        router = fetch.vector(s.router_weight)
+        if s.shared_gate_weight:        # one more row of the router's product
+            router = torch.cat([router, fetch.vector(s.shared_gate_weight)], dim=0)
+        self.w_router = fetch.to_device(router)
+        self.correction = fetch.to_device(fetch.vector(s.correction_weight)) if s.correction_weight else None
         if (getattr(fetch, "tiled_copies", False) and self.w_up.dtype == torch.bfloat16 and s.intermediate_size % 32 == 0
                 and s.hidden_size % 32 == 0):
             # a band of 16 rows never holds rows of two experts (nor gate rows beside up rows)
@@ -111,23 +127,17 @@ class MixtureOfExperts:
         n = h.shape[0]
         ids = ctx.buffer("moe_ids", (n, s.top), torch.int32)
         weights = ctx.buffer("moe_weights", (n, s.top), torch.float32)
+        gates = ctx.buffer("moe_gates", (n,), torch.float32) if s.shared_gate_weight else None
         ops.moe_route(h, self.w_router, ids, weights, groups=s.num_groups, keep=s.keep_groups, eps=s.weight_eps,
-                      scoring=s.scoring, normalize=s.normalize)
+                      scoring=s.scoring, normalize=s.normalize, correction=self.correction, group_best=s.group_best, gates=gates)
         rows = ops.moe_tile_rows(n * s.top, s.num_experts, h.dtype, s.hidden_size, s.intermediate_size)
         plan = ctx.buffer("moe_plan", (ops.moe_plan_size(n * s.top, s.num_experts, rows),), torch.int32)
         ops.moe_plan(ids, plan, s.num_experts, rows)
         act = ctx.buffer("moe_act", (n * s.top, s.intermediate_size), h.dtype)
         ops.moe_experts_up(h, self.w_up, plan, act, s.top, s.activation, rows, self.t_up,
                            in_weights=weights if s.weight_on_input else None)
-        out = ctx.buffer("moe_out", (s.top + (1 if self.shared is not None else 0), n, s.hidden_size), torch.float32)
-        ops.moe_experts_down(act, self.w_down, plan, weights, out[:s.top], rows, self.t_down, weighted=not s.weight_on_input)
-        if self.shared is not None:
-            # the expert every token uses: its product's float32 sums are the stack's last slice
-            last = self.shared.forward(ctx, h)
-            if h.dtype == torch.float32 or n <= 64:
-                ops.linear(last.x, last.weight, out[s.top], last.tiles)
-            else:
-                # many rows: the product as every other of this size is made (in the activation type), then into its slice
-                out[s.top].zero_()
-                ops.stream_add(out[s.top], delta=last.make(ctx))
-        return out
+        out = ctx.buffer("moe_out", (s.top, n, s.hidden_size), torch.float32)
+        ops.moe_experts_down(act, self.w_down, plan, weights, out, rows, self.t_down, weighted=not s.weight_on_input)
+        if self.shared is None:
+            return out
+        return TwoTerms(out, self.shared.forward(ctx, h), gates)

@@ -82,7 +82,9 @@ class AttentionSpec(MixerSpec):
     `q_head_norm_weight` / `k_head_norm_weight` with `head_norm_eps`: before the rotation every query head and
     every key head passes an RMS norm over its own elements with a weight of head_dim numbers that the heads
     share.  `sink_weight`: the term in the softmax's denominator is exp(sink_h) of a learned number a head
-    (a tensor [num_heads]) instead of the constant `sink`."""
+    (a tensor [num_heads]) instead of the constant `sink`.
+    `q_temperature` = (coef, every): behind rotation and norm a query at position p is multiplied by
+    1 + coef * ln(floor((p + 1) / every) + 1)."""
     kind: str = "attention"
     hidden_size: int = 0
     num_heads: int = 0
@@ -119,6 +121,7 @@ class AttentionSpec(MixerSpec):
     k_head_norm_weight: Optional[str] = None
     head_norm_eps: Optional[float] = None
     sink_weight: Optional[str] = None
+    q_temperature: Optional[tuple] = None
 
 
 @dataclass(frozen=True)
@@ -242,6 +245,48 @@ class MatrixMemorySpec(MixerSpec):
 
 
 @dataclass(frozen=True)
+class DeltaRuleSpec(MixerSpec):
+    """A recurrent mixer whose state is a matrix a head, S [head_dim, value_dim] in float32, corrected by what it
+    already answers (the gated delta rule) and with a decay a head and key channel:
+        q = W_q h, k = W_k h (num_kv_heads heads of head_dim), v = W_v h (num_heads heads of value_dim); each passes a short
+        causal convolution per channel (`conv_taps` taps, no bias) and silu; q and k become unit vectors a head
+        (x / sqrt(sum(x^2) + unit_eps)), q times q_scale; head h uses q and k head h // (num_heads // num_kv_heads)
+        beta = sigmoid(W_b h), a number a head;  g = exp(-exp(a_log) softplus(W_a2 (W_a1 h) + dt_bias)), one a head and channel
+        S = diag(g) S;  u = beta (v - S^T k);  S = S + k u^T;  o = S^T q
+    Then every head's o is divided by its root mean square (`norm_eps` inside the root), multiplied by `norm_weight`
+    (value_dim numbers that the heads share) and by sigmoid(W_g2 (W_g1 h)), and the heads are projected by W_o.
+    The two inner sizes (rows of W_a1 and of W_g1) are the checkpoint's; `decay_rank` and `gate_rank` are what the
+    random-weights mode draws.  A request carries S and the convolutions' last conv_taps - 1 inputs."""
+    kind: str = "delta_rule"
+    hidden_size: int = 0
+    num_heads: int = 0
+    num_kv_heads: int = 0
+    head_dim: int = 0
+    value_dim: int = 0
+    conv_taps: int = 4
+    q_scale: float = 1.0
+    unit_eps: float = 1e-6
+    norm_eps: float = 1e-6
+    decay_rank: int = 16
+    gate_rank: int = 16
+    q_weight: str = ""
+    k_weight: str = ""
+    v_weight: str = ""
+    q_conv_weight: str = ""
+    k_conv_weight: str = ""
+    v_conv_weight: str = ""
+    b_weight: str = ""
+    a1_weight: str = ""
+    a2_weight: str = ""
+    a_log: str = ""
+    dt_bias: str = ""
+    g1_weight: str = ""
+    g2_weight: str = ""
+    norm_weight: str = ""
+    o_weight: str = ""
+
+
+@dataclass(frozen=True)
 class SideBySideSpec(MixerSpec):
     """Two mixers that read the same input; the result is the sum of theirs (each weighs its own with its
     `output_scale`).  At most one of the two pages a cache and at most one carries a state."""
@@ -290,6 +335,17 @@ class GatedMLPSpec(FeedForwardSpec):
 
 
 @dataclass(frozen=True)
+class MLPSpec(FeedForwardSpec):
+    """down(act(up(x))) without a gate and without biases; `activation` "squared_relu", "gelu_tanh" or "silu"."""
+    kind: str = "mlp"
+    hidden_size: int = 0
+    intermediate_size: int = 0
+    activation: str = "squared_relu"
+    up_weight: str = ""
+    down_weight: str = ""
+
+
+@dataclass(frozen=True)
 class MixtureOfExpertsSpec(FeedForwardSpec):
     """`num_experts` gated feed-forwards without biases, down_e(act(gate_e(x)) * up_e(x)), of which a token
     uses `top`.  Router: z = W_router x in float32, s = softmax(z) over all experts.  The experts form
@@ -300,7 +356,9 @@ class MixtureOfExpertsSpec(FeedForwardSpec):
     expert's tensors.  `scoring` "sigmoid": s = sigmoid(z), every expert by itself.  `normalize` False: the
     weights are the chosen s themselves.  `weight_on_input`: the weight multiplies the expert's input instead of
     its output, y = sum of expert_e(w_e x).  `shared`: one more gated feed-forward that every token uses, added to
-    the experts' sum."""
+    the experts' sum; `shared_gate_weight` ([1, hidden]): its result is first multiplied by sigmoid(W x), a number a token.
+    `correction_weight` ([num_experts]): every choice (of groups and of experts) is made by c = s + correction; the weights
+    come of s alone.  `group_best` 2: a group's score is the sum of its two largest c."""
     kind: str = "mixture_of_experts"
     hidden_size: int = 0
     intermediate_size: int = 0
@@ -319,6 +377,9 @@ class MixtureOfExpertsSpec(FeedForwardSpec):
     normalize: bool = True
     weight_on_input: bool = False
     shared: Optional[GatedMLPSpec] = None
+    shared_gate_weight: Optional[str] = None
+    correction_weight: Optional[str] = None
+    group_best: int = 1
 
 
 @dataclass(frozen=True)
@@ -342,7 +403,9 @@ class BlockSpec:
     feed-forward has neither of its norms), then the layer's token input (`side`), if it has one.
     "post_norm": x += post(mixer(x)); x += post(ffn(x)): the sublayers read the stream itself and the only norms
     stand behind them (`mixer_norm` and `feed_forward_norm` are None).  With `mixer_input_conv` /
-    `feed_forward_input_conv` what a sublayer reads first passes a short convolution over time (`InputConvSpec`)."""
+    `feed_forward_input_conv` what a sublayer reads first passes a short convolution over time (`InputConvSpec`).
+    "norm_of_sum": x = post(w x + mixer(x)); x = post(w x + ffn(x)) with w = `stream_weight`: the sublayers read the
+    stream itself, and the norm behind each takes the sum (the names of the norms are those of "post_norm")."""
     mixer: MixerSpec
     feed_forward: Optional[FeedForwardSpec]
     mixer_norm: Optional[NormSpec]
@@ -353,6 +416,7 @@ class BlockSpec:
     side: Optional[TokenSideSpec] = None
     mixer_input_conv: Optional[InputConvSpec] = None
     feed_forward_input_conv: Optional[InputConvSpec] = None
+    stream_weight: float = 1.0
 
 
 @dataclass(frozen=True)

@@ -39,6 +39,14 @@ class ExpectedTensor:
     optional: bool = False
     # how the random-weights mode draws it: "weight" (normal, std) or "norm" (normal, norm_std)
     init: str = "weight"
+    # axes whose size is the checkpoint's to say: `shape` then holds what the random-weights mode draws there
+    free_axes: tuple = ()
+
+    def takes(self, shape: tuple) -> bool:
+        """Whether a stored tensor of `shape` is this one."""
+        return len(shape) == len(self.shape) and all(
+            stored == own or (axis in self.free_axes and stored > 0)
+            for axis, (stored, own) in enumerate(zip(shape, self.shape)))
 
 
 _FLOATS = (torch.float32, torch.bfloat16, torch.float16, torch.float64)
@@ -104,7 +112,7 @@ class Checkpoint:
                     missing.append(name)
                 continue
             shape = self.shape(name)
-            if tuple(shape) != tuple(exp.shape):
+            if not exp.takes(tuple(shape)):
                 wrong_shape.append((name, tuple(shape), tuple(exp.shape)))
             dt = self.stored_dtype(name)
             ok = dt in _INTS if exp.role == "table" else dt in _FLOATS
