@@ -10,6 +10,21 @@
 #include "common.h"
 #include "short_conv.h"
 
+// The sum over 32 lanes, within each half of the wavefront, in every lane of it; and the value of the lane 32 apart.
+__device__ __forceinline__ float row_halves_sum(float v) {
+    v = sum_across(v, 16);
+    v += row_permuted<0x128>(v);
+    v += row_permuted<0x124>(v);
+    v += row_permuted<0x4E>(v);
+    v += row_permuted<0xB1>(v);
+    return v;
+}
+__device__ __forceinline__ float from_other_half(float v) {
+    float a, b;                                  // the lower half's value and the upper half's, in both
+    swap_halves(v, 32, a, b);
+    return threadIdx.x % kWave < 32 ? b : a;
+}
+
 __device__ __forceinline__ float delta_softplus(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
 
 // ---- what the recurrence reads, from a token's projections:
@@ -116,6 +131,128 @@ delta_inputs_kernel(const T* __restrict__ xqkv, long long x_stride, const T* __r
     }
 }
 
+// The same with four consecutive channels a lane (D, P, the rows' strides and the carried rows' place are multiples of
+// four): lanes 0 .. 31 of a group's wavefront hold q, lanes 32 .. 63 k.
+template <typename T> struct alignas(4 * sizeof(T)) DeltaFour { T v[4]; };
+
+template <typename T, bool CARRY>
+__device__ __forceinline__ float4 short_conv_four(const T* now, long long stride, int local, float* carried, const float* w,
+                                                  int channels, int taps, int c) {
+    const DeltaFour<T> mine = *reinterpret_cast<const DeltaFour<T>*>(now + c);
+    float4 acc = make_float4(0.f, 0.f, 0.f, 0.f);
+    auto add = [&](const float4 wv, const float4 x) {
+        acc.x = fmaf(wv.x, x.x, acc.x);
+        acc.y = fmaf(wv.y, x.y, acc.y);
+        acc.z = fmaf(wv.z, x.z, acc.z);
+        acc.w = fmaf(wv.w, x.w, acc.w);
+    };
+#pragma unroll 4
+    for (int k = 0; k + 1 < taps; ++k) {
+        const int back = taps - 1 - k;
+        float4 x;
+        if (CARRY || local < back) {
+            x = *reinterpret_cast<const float4*>(carried + static_cast<size_t>(k + (CARRY ? 0 : local)) * channels + c);
+            if (CARRY && k > 0) *reinterpret_cast<float4*>(carried + static_cast<size_t>(k - 1) * channels + c) = x;
+        } else {
+            const DeltaFour<T> e = *reinterpret_cast<const DeltaFour<T>*>(now + c - back * stride);
+            x = make_float4(to_float(e.v[0]), to_float(e.v[1]), to_float(e.v[2]), to_float(e.v[3]));
+        }
+        add(*reinterpret_cast<const float4*>(w + static_cast<size_t>(k) * channels + c), x);
+    }
+    const float4 x = make_float4(to_float(mine.v[0]), to_float(mine.v[1]), to_float(mine.v[2]), to_float(mine.v[3]));
+    if (CARRY && taps > 1) *reinterpret_cast<float4*>(carried + static_cast<size_t>(taps - 2) * channels + c) = x;
+    add(*reinterpret_cast<const float4*>(w + static_cast<size_t>(taps - 1) * channels + c), x);
+    acc.x /= 1.f + expf(-acc.x);
+    acc.y /= 1.f + expf(-acc.y);
+    acc.z /= 1.f + expf(-acc.z);
+    acc.w /= 1.f + expf(-acc.w);
+    return acc;
+}
+
+__device__ __forceinline__ float dot4(const float4 a, const float4 b) { return fmaf(a.w, b.w, fmaf(a.z, b.z, fmaf(a.y, b.y, a.x * b.x))); }
+
+template <typename T, bool CARRY>
+__global__ void __launch_bounds__(kWave * kDeltaWaves)
+delta_inputs_four_kernel(const T* __restrict__ xqkv, long long x_stride, const T* __restrict__ z, long long z_stride,
+                         const T* __restrict__ b, long long b_stride, T* __restrict__ v, DeltaInputs a) {
+    const int token = blockIdx.x;
+    const int lane = threadIdx.x % kWave, wave = threadIdx.x / kWave;
+    const int seg = a.token_segment[token];
+    const int local = token - a.seg_q_start[seg];
+    const int channels = 2 * a.groups * a.d + a.heads * a.p_dim;
+    float* carried = a.state + static_cast<size_t>(a.state_slots[seg]) * a.state_stride + a.carried_offset;
+    const T* xt = xqkv + static_cast<size_t>(token) * x_stride;
+    auto convolved = [&](int c) { return short_conv_four<T, CARRY>(xt, x_stride, local, carried, a.conv_w, channels, a.taps, c); };
+    int unit = blockIdx.y * kDeltaWaves + wave;
+    if (unit < a.groups) {
+        constexpr int kPer = 2;                  // heads of up to 32 * 4 * 2 channels
+        const int half = lane / 32;              // 0: q, 1: k
+        float4 x[kPer];
+        float ss = 0.f;
+#pragma unroll
+        for (int j = 0; j < kPer; ++j) {
+            const int i = 4 * (lane % 32 + 32 * j);
+            x[j] = make_float4(0.f, 0.f, 0.f, 0.f);
+            if (i < a.d) x[j] = convolved((half * a.groups + unit) * a.d + i);
+            ss += dot4(x[j], x[j]);
+        }
+        ss = row_halves_sum(ss);
+        const float inv = (half ? 1.f : a.q_scale) / sqrtf(ss + a.unit_eps);
+        float* out = a.qk + (static_cast<size_t>(half) * a.tokens + token) * a.groups * a.dp + static_cast<size_t>(unit) * a.dp;
+        float dot = 0.f;
+#pragma unroll
+        for (int j = 0; j < kPer; ++j) {
+            const int i = 4 * (lane % 32 + 32 * j);
+            x[j].x *= inv;
+            x[j].y *= inv;
+            x[j].z *= inv;
+            x[j].w *= inv;
+            const float4 other = make_float4(from_other_half(x[j].x), from_other_half(x[j].y), from_other_half(x[j].z),
+                                             from_other_half(x[j].w));
+            dot += dot4(x[j], other);
+            if (i < a.d) *reinterpret_cast<float4*>(out + i) = x[j];
+        }
+        dot = row_halves_sum(dot);
+        if (lane == 0) a.kq[static_cast<size_t>(token) * a.groups + unit] = dot;
+        return;
+    }
+    unit -= a.groups;
+    const int v_width = a.heads * a.p_dim, f_width = a.heads * a.d;
+#pragma unroll
+    for (int j = 0; j < kDeltaPer; ++j) {
+        int e = (unit * kWave * kDeltaPer + kWave * j + lane) * 4;
+        if (e < v_width) {
+            const float4 x = convolved(2 * a.groups * a.d + e);
+            DeltaFour<T> r;
+            r.v[0] = from_float<T>(x.x);
+            r.v[1] = from_float<T>(x.y);
+            r.v[2] = from_float<T>(x.z);
+            r.v[3] = from_float<T>(x.w);
+            *reinterpret_cast<DeltaFour<T>*>(v + static_cast<size_t>(token) * v_width + e) = r;
+            continue;
+        }
+        e -= v_width;
+        if (e < f_width) {
+            const float rate = a.rate[e / a.d];
+            const DeltaFour<T> zv = *reinterpret_cast<const DeltaFour<T>*>(z + static_cast<size_t>(token) * z_stride + e);
+            const float4 bias = *reinterpret_cast<const float4*>(a.dt_bias + e);
+            float4 r;
+            r.x = expf(-rate * delta_softplus(to_float(zv.v[0]) + bias.x));
+            r.y = expf(-rate * delta_softplus(to_float(zv.v[1]) + bias.y));
+            r.z = expf(-rate * delta_softplus(to_float(zv.v[2]) + bias.z));
+            r.w = expf(-rate * delta_softplus(to_float(zv.v[3]) + bias.w));
+            *reinterpret_cast<float4*>(a.f + static_cast<size_t>(token) * f_width + e) = r;
+            continue;
+        }
+        e -= f_width;
+#pragma unroll
+        for (int u = 0; u < 4; ++u)
+            if (e + u < a.heads)
+                a.beta[static_cast<size_t>(token) * a.heads + e + u] =
+                    1.f / (1.f + expf(-to_float(b[static_cast<size_t>(token) * b_stride + e + u])));
+    }
+}
+
 WLLM_API int wllm_delta_inputs(const void* xqkv, long long x_stride, const void* z, long long z_stride, const void* b,
                                long long b_stride, const float* conv_w, const float* rate, const float* dt_bias, float* state,
                                long long state_stride, long long carried_offset, const int* token_segment, const int* seg_q_start,
@@ -132,6 +269,25 @@ WLLM_API int wllm_delta_inputs(const void* xqkv, long long x_stride, const void*
     if (pieces > 65535) return -1;
     const DeltaInputs a{conv_w, state, state_stride, carried_offset, token_segment, seg_q_start, state_slots, rate, dt_bias, qk, kq, f,
                         beta, q_scale, unit_eps, tokens, heads, groups, d, dp, p_dim, taps};
+    const size_t four_bytes = 4 * (is_bf16 ? 2 : 4);
+    const bool four = d % 4 == 0 && p_dim % 4 == 0 && x_stride % 4 == 0 && z_stride % 4 == 0 && state_stride % 4 == 0 &&
+                      carried_offset % 4 == 0 && reinterpret_cast<uintptr_t>(xqkv) % four_bytes == 0 &&
+                      reinterpret_cast<uintptr_t>(z) % four_bytes == 0 && reinterpret_cast<uintptr_t>(v) % four_bytes == 0 &&
+                      reinterpret_cast<uintptr_t>(conv_w) % 16 == 0 && reinterpret_cast<uintptr_t>(dt_bias) % 16 == 0 &&
+                      reinterpret_cast<uintptr_t>(state) % 16 == 0 && reinterpret_cast<uintptr_t>(qk) % 16 == 0 &&
+                      reinterpret_cast<uintptr_t>(f) % 16 == 0;
+    if (four) {
+        const long long fours = rest / 4 + 1;    // (beta's last four may be partly there)
+        const long long four_units = groups + (fours + kWave * kDeltaPer - 1) / (kWave * kDeltaPer);
+        const dim3 four_grid(tokens, static_cast<unsigned>((four_units + kDeltaWaves - 1) / kDeltaWaves));
+#define LAUNCH(T, CARRY)                                                                                                \
+    delta_inputs_four_kernel<T, CARRY><<<four_grid, kWave * kDeltaWaves, 0, stream>>>(                                  \
+        static_cast<const T*>(xqkv), x_stride, static_cast<const T*>(z), z_stride, static_cast<const T*>(b), b_stride,  \
+        static_cast<T*>(v), a)
+        if (is_bf16) { if (single_tokens) LAUNCH(bf16, true); else LAUNCH(bf16, false); }
+        else { if (single_tokens) LAUNCH(float, true); else LAUNCH(float, false); }
+#undef LAUNCH
+    } else {
     const dim3 grid(tokens, static_cast<unsigned>(pieces));
 #define LAUNCH(T, CARRY)                                                                                                \
     delta_inputs_kernel<T, CARRY><<<grid, kWave * kDeltaWaves, 0, stream>>>(                                            \
@@ -140,6 +296,7 @@ WLLM_API int wllm_delta_inputs(const void* xqkv, long long x_stride, const void*
     if (is_bf16) { if (single_tokens) LAUNCH(bf16, true); else LAUNCH(bf16, false); }
     else { if (single_tokens) LAUNCH(float, true); else LAUNCH(float, false); }
 #undef LAUNCH
+    }
     if (const int err = launch_status()) return err;
     if (taps == 1 || single_tokens) return 0;
     const int channels = 2 * groups * d + heads * p_dim;
@@ -241,37 +398,51 @@ delta_scan_kernel(const float* __restrict__ qk, const float* __restrict__ kq, co
         }
     };
     float kept = 0.f;                                        // lane sl of a column keeps the result of token sl of the 16
-    auto token = [&](int t) {
-        float4 kt[R];
-        float seen[2] = {0.f, 0.f}, read[2] = {0.f, 0.f};    // two chains each
+    struct Operands {
+        float4 k[R], q[R], f[R];
+        float v, beta, kq;
+    };
+    auto load = [&](int t) {
+        Operands o;
 #pragma unroll
         for (int j = 0; j < R; ++j) {
             const int at = t * kRow + 64 * j + 4 * sl;
-            kt[j] = *reinterpret_cast<const float4*>(k_s + at);
-            const float4 qt = *reinterpret_cast<const float4*>(q_s + at), ft = *reinterpret_cast<const float4*>(f_s + at);
-            s[j].x *= ft.x;
-            s[j].y *= ft.y;
-            s[j].z *= ft.z;
-            s[j].w *= ft.w;
-            seen[0] = fmaf(s[j].x, kt[j].x, seen[0]);
-            seen[1] = fmaf(s[j].y, kt[j].y, seen[1]);
-            seen[0] = fmaf(s[j].z, kt[j].z, seen[0]);
-            seen[1] = fmaf(s[j].w, kt[j].w, seen[1]);
-            read[0] = fmaf(s[j].x, qt.x, read[0]);
-            read[1] = fmaf(s[j].y, qt.y, read[1]);
-            read[0] = fmaf(s[j].z, qt.z, read[0]);
-            read[1] = fmaf(s[j].w, qt.w, read[1]);
+            o.k[j] = *reinterpret_cast<const float4*>(k_s + at);
+            o.q[j] = *reinterpret_cast<const float4*>(q_s + at);
+            o.f[j] = *reinterpret_cast<const float4*>(f_s + at);
         }
-        const float u = beta_s[t] * (v_s[t * kScanCols + col] - row_sum(seen[0] + seen[1]));
-        const float o = fmaf(u, kq_s[t], row_sum(read[0] + read[1]));
+        o.v = v_s[t * kScanCols + col];
+        o.beta = beta_s[t];
+        o.kq = kq_s[t];
+        return o;
+    };
+    auto token = [&](int t, const Operands& o) {
+        float seen[2] = {0.f, 0.f}, read[2] = {0.f, 0.f};    // two chains each
 #pragma unroll
         for (int j = 0; j < R; ++j) {
-            s[j].x = fmaf(kt[j].x, u, s[j].x);
-            s[j].y = fmaf(kt[j].y, u, s[j].y);
-            s[j].z = fmaf(kt[j].z, u, s[j].z);
-            s[j].w = fmaf(kt[j].w, u, s[j].w);
+            s[j].x *= o.f[j].x;
+            s[j].y *= o.f[j].y;
+            s[j].z *= o.f[j].z;
+            s[j].w *= o.f[j].w;
+            seen[0] = fmaf(s[j].x, o.k[j].x, seen[0]);
+            seen[1] = fmaf(s[j].y, o.k[j].y, seen[1]);
+            seen[0] = fmaf(s[j].z, o.k[j].z, seen[0]);
+            seen[1] = fmaf(s[j].w, o.k[j].w, seen[1]);
+            read[0] = fmaf(s[j].x, o.q[j].x, read[0]);
+            read[1] = fmaf(s[j].y, o.q[j].y, read[1]);
+            read[0] = fmaf(s[j].z, o.q[j].z, read[0]);
+            read[1] = fmaf(s[j].w, o.q[j].w, read[1]);
         }
-        if (sl == t) kept = o;
+        const float u = o.beta * (o.v - row_sum(seen[0] + seen[1]));
+        const float out = fmaf(u, o.kq, row_sum(read[0] + read[1]));
+#pragma unroll
+        for (int j = 0; j < R; ++j) {
+            s[j].x = fmaf(o.k[j].x, u, s[j].x);
+            s[j].y = fmaf(o.k[j].y, u, s[j].y);
+            s[j].z = fmaf(o.k[j].z, u, s[j].z);
+            s[j].w = fmaf(o.k[j].w, u, s[j].w);
+        }
+        if (sl == t) kept = out;
     };
     fetch(0);
     for (int t0 = 0; t0 < q_len; t0 += kScanTokens) {
@@ -280,10 +451,16 @@ delta_scan_kernel(const float* __restrict__ qk, const float* __restrict__ kq, co
         __syncthreads();
         if (t0 + kScanTokens < q_len) fetch(t0 + kScanTokens);
         if (count == kScanTokens) {
+            Operands now = load(0);
 #pragma unroll
-            for (int t = 0; t < kScanTokens; ++t) token(t);
+            for (int t = 0; t < kScanTokens; ++t) {
+                const Operands next = load(t + 1 < kScanTokens ? t + 1 : t);      // on their way while this token is worked on
+                __builtin_amdgcn_sched_barrier(0);
+                token(t, now);
+                now = next;
+            }
         } else {
-            for (int t = 0; t < count; ++t) token(t);
+            for (int t = 0; t < count; ++t) token(t, load(t));
         }
         if (live && sl < count)
             y[static_cast<size_t>(q_start + t0 + sl) * heads * p_dim + static_cast<size_t>(h) * p_dim + p] = kept;
