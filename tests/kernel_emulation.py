@@ -515,13 +515,25 @@ class EmulatedKernels:
         f.view(n, heads, dp)[..., :head_dim] = torch.exp(-rate.to(acc)[:, None] * dt).float()
         beta.copy_(torch.sigmoid(b.to(acc)).float())
 
-    def delta_scan(self, qk, kq, f, beta, v, state, seg_q_start, seg_q_len, state_slots, y, heads, groups, head_dim, value_dim):
+    def delta_chunk_scan(self, qk, f, beta, v, state, token_segment, seg_q_start, seg_q_len, state_slots, y, chunks, heads, groups,
+                         head_dim, value_dim, from_tokens):
+        self._count("delta_chunk_scan")
+        chunks.fill_(float("nan"))
+        self._delta_walk(qk, f, beta, v, state, seg_q_start, seg_q_len, state_slots, y, heads, groups, value_dim, from_tokens, 1 << 31)
+
+    def delta_scan(self, qk, kq, f, beta, v, state, seg_q_start, seg_q_len, state_slots, y, heads, groups, head_dim, value_dim,
+                   shorter_than=1 << 31):
         self._count("delta_scan")
+        self._delta_walk(qk, f, beta, v, state, seg_q_start, seg_q_len, state_slots, y, heads, groups, value_dim, 0, shorter_than)
+
+    def _delta_walk(self, qk, f, beta, v, state, seg_q_start, seg_q_len, state_slots, y, heads, groups, value_dim, least, below):
         acc = self.acc
         dp, per = f.shape[1] // heads, heads // groups
         size = heads * value_dim * dp
         for s in range(seg_q_start.shape[0]):
             q0, ql, slot = int(seg_q_start[s]), int(seg_q_len[s]), int(state_slots[s])
+            if not least <= ql < below:
+                continue
             S = state[slot, :size].to(acc).view(heads, value_dim, dp).clone()
             for t in range(q0, q0 + ql):
                 q, k = (qk[i, t].to(acc).view(groups, dp).repeat_interleave(per, dim=0) for i in range(2))

@@ -33,7 +33,13 @@ SHARP_BOUND = {torch.float32: dict(relative=6e-4, times=6.0), torch.bfloat16: di
 
 
 def check_rows(got, folder, requests, exact, dtype, sharp=False):
-    return compare_with_rounding(got, exact, rounding_noise(folder, requests, dtype, exact), **(SHARP_BOUND if sharp else BOUND)[dtype])
+    noise, bound = rounding_noise(folder, requests, dtype, exact), dict((SHARP_BOUND if sharp else BOUND)[dtype])
+    if dtype == torch.bfloat16:
+        # where the plain implementation's own rounding chooses other experts for many rows, the engine's may for as many others
+        far = [float(noise[rid][pos]) > bound["relative"] * (exact[rid][pos] - exact[rid][pos].mean()).pow(2).mean().sqrt().item()
+               for rid, pos in got]
+        bound["outliers"] = max(bound["outliers"], 1.5 * sum(far) / len(far))
+    return compare_with_rounding(got, exact, noise, **bound)
 
 
 def close(got, ref, dtype, what="", scale=1.0):
@@ -248,9 +254,19 @@ DELTA_SIZES = [(4, 2, 16, 32, 4), (3, 1, 10, 6, 1), (1, 1, 130, 5, 7), (4, 2, 7,
                (3, 3, 192, 12, 5), (5, 5, 4, 130, 2), (2, 2, 100, 33, 4)]
 
 
+def _walk(chunked, qk, kq, f, beta, v, state, of, seg, y, sizes):
+    """The recurrence over a step: token by token, or (the segments of `chunked` tokens and more) in chunks."""
+    if chunked:
+        n = v.shape[0]
+        chunks = torch.full((ops.delta_chunk_size(n, seg[0].shape[0], sizes["heads"], sizes["head_dim"]),), float("nan"), device=DEV)
+        ops.delta_chunk_scan(qk, f, beta, v, state, of, *seg, y, chunks, from_tokens=chunked, **sizes)
+    ops.delta_scan(qk, kq, f, beta, v, state, *seg, y, shorter_than=chunked, **sizes)
+
+
 @pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("chunked", [None, 16, 40])
 @pytest.mark.parametrize("H,G,d,dv,taps", DELTA_SIZES)
-def test_the_delta_rule_whole_and_token_by_token(dtype, H, G, d, dv, taps):
+def test_the_delta_rule_whole_and_token_by_token(dtype, H, G, d, dv, taps, chunked):
     """The convolutions, unit vectors, decays, step sizes, the recurrence and the gated norm, over a prompt and over the
     same prompt in pieces down to single tokens, through a state row that lies beside rows that must not change."""
     g = torch.Generator().manual_seed(H * d + dv)
@@ -276,8 +292,7 @@ def test_the_delta_rule_whole_and_token_by_token(dtype, H, G, d, dv, taps):
     wide = torch.full((T, -(-width // 8) * 8 + 8), float("nan"), dtype=dtype)
     wide[:, 8:8 + width] = row
     wide = wide.to(DEV)
-    rows_of = {}
-    for pieces in ([1000], [64, 33], [16, 5, 2, 1, 33], [1]):
+    for pieces in ([1000], [64, 33], [16, 5, 2, 1, 33, 17]) + (() if chunked else ([1],)):
         state = torch.full((5, total), 9.0, device=DEV)
         state[2] = 0.0
         outs = []
@@ -290,30 +305,30 @@ def test_the_delta_rule_whole_and_token_by_token(dtype, H, G, d, dv, taps):
             v = nan(n, v_w).to(dtype)
             ops.delta_inputs(r[:, :channels], z[lo:hi], r[:, b_at:b_at + H], conv, rate, bias, state, memory, _i32([0] * n), *seg, qk, kq,
                              v, f, beta, q_scale=d ** -0.5, unit_eps=1e-6, single_tokens=n == 1, **sizes)
-            ops.delta_scan(qk, kq, f, beta, v, state, *seg, y, **sizes)
+            _walk(chunked, qk, kq, f, beta, v, state, _i32([0] * n), seg, y, sizes)
             out = torch.zeros(n, v_w, dtype=dtype, device=DEV)
             ops.head_norm_gate(y, gate[lo:hi], norm, out, heads=H, eps=eps, activation="sigmoid")
             outs.append(out.cpu())
         got = torch.cat(outs)
-        rows_of[tuple(pieces)] = got
         for t in range(T):
             close(got[t], want[t], dtype, f"token {t}, pieces {pieces}", scale=3.0 + 8.0 * float(noise[t]) / 3e-5)
         assert (state[[0, 1, 3, 4]] == 9.0).all()
 
 
-@pytest.mark.parametrize("H,G,d,dv,taps", [(4, 2, 16, 32, 4), (2, 1, 128, 128, 4), (3, 1, 10, 6, 3), (1, 1, 256, 40, 2)])
-def test_a_batch_of_unequal_requests_against_each_alone(H, G, d, dv, taps):
+@pytest.mark.parametrize("chunked", [None, 16, 33])
+@pytest.mark.parametrize("H,G,d,dv,taps", [(4, 2, 16, 32, 4), (2, 1, 128, 128, 4), (3, 1, 10, 6, 3), (1, 1, 256, 40, 2), (2, 2, 192, 17, 4)])
+def test_a_batch_of_unequal_requests_against_each_alone(H, G, d, dv, taps, chunked):
     """Segments of a few tokens to some hundred side by side, in slots of any order, each with a memory and carried rows
     of its own: the results and what is left behind are those of each request alone."""
     g = torch.Generator().manual_seed(d)
-    lengths, slots = [1, 2, 70, 1, 17, 200, 16, 33], [3, 0, 7, 1, 5, 2, 8, 6]
+    lengths, slots = [1, 2, 70, 1, 17, 200, 16, 33, 15, 16], [3, 0, 7, 1, 5, 2, 8, 6, 10, 9]
     n, channels = sum(lengths), 2 * G * d + H * dv
     dp, memory = ops.delta_padded(d), ops.delta_state_size(H, d, dv)
     total = -(-(memory + (taps - 1) * channels) // 4) * 4
     x, z, b = torch.randn(n, channels, generator=g).to(DEV), torch.randn(n, H * d, generator=g).to(DEV), torch.randn(n, H, generator=g).to(DEV)
     conv, rate = torch.randn(taps, channels, generator=g).to(DEV), (torch.rand(H, generator=g) + 0.1).to(DEV)
     bias = (-3.0 + torch.randn(H * d, generator=g)).to(DEV)
-    state0 = torch.randn(9, total, generator=g).to(DEV) * 0.3
+    state0 = torch.randn(11, total, generator=g).to(DEV) * 0.3
     sizes = dict(heads=H, groups=G, head_dim=d, value_dim=dv)
 
     def run(x, z, b, lengths, slots, state):
@@ -324,10 +339,10 @@ def test_a_batch_of_unequal_requests_against_each_alone(H, G, d, dv, taps):
         e = lambda *s: torch.zeros(s, device=DEV)
         qk, kq, f, beta, y, v = e(2, n, G * dp), e(n, G), e(n, H * dp), e(n, H), e(n, H * dv), e(n, H * dv)
         ops.delta_inputs(x, z, b, conv, rate, bias, state, memory, of, *seg, qk, kq, v, f, beta, q_scale=d ** -0.5, unit_eps=1e-6, **sizes)
-        ops.delta_scan(qk, kq, f, beta, v, state, *seg, y, **sizes)
+        _walk(chunked, qk, kq, f, beta, v, state, of, seg, y, sizes)
         return y
 
-    pad = state0[:, :memory].view(9, H, dv, dp)
+    pad = state0[:, :memory].view(11, H, dv, dp)
     pad[..., d:] = 0.0                          # what lies behind a head's channels is zero
     together = state0.clone()
     y = run(x, z, b, lengths, slots, together)

@@ -336,7 +336,7 @@ __global__ void __launch_bounds__(kScanThreads)
 delta_scan_kernel(const float* __restrict__ qk, const float* __restrict__ kq, const float* __restrict__ f,
                   const float* __restrict__ beta, const T* __restrict__ v, float* __restrict__ state, long long state_stride,
                   const int* __restrict__ seg_q_start, const int* __restrict__ seg_q_len, const int* __restrict__ state_slots,
-                  float* __restrict__ y, int tokens, int heads, int groups, int dp, int p_dim) {
+                  float* __restrict__ y, int tokens, int heads, int groups, int dp, int p_dim, int shorter_than) {
     constexpr int kRow = 64 * R;                             // a token's k (q, f) in shared memory: DP channels and zeros
     constexpr int kFours = kScanTokens * kRow / 4 / kScanThreads;      // groups of four of each that a thread stages: R
     __shared__ __align__(16) float q_s[kScanTokens * kRow], k_s[kScanTokens * kRow], f_s[kScanTokens * kRow];
@@ -344,7 +344,7 @@ delta_scan_kernel(const float* __restrict__ qk, const float* __restrict__ kq, co
     __shared__ float beta_s[kScanTokens], kq_s[kScanTokens];
     const int h = blockIdx.x, seg = blockIdx.y, p0 = blockIdx.z * kScanCols;
     const int q_len = seg_q_len[seg], q_start = seg_q_start[seg];
-    if (q_len <= 0) return;
+    if (q_len <= 0 || q_len >= shorter_than) return;
     const int tid = threadIdx.x, lane = tid % kWave, wave = tid / kWave;
     const int sl = lane % kScanLanes, col = wave * (kWave / kScanLanes) + lane / kScanLanes;
     const int p = p0 + col;
@@ -475,9 +475,11 @@ delta_scan_kernel(const float* __restrict__ qk, const float* __restrict__ kq, co
     }
 }
 
+// Segments of `shorter_than` tokens and more are left alone (a caller that takes none of them away passes INT_MAX).
 WLLM_API int wllm_delta_scan(const float* qk, const float* kq, const float* f, const float* beta, const void* v, float* state,
                              long long state_stride, const int* seg_q_start, const int* seg_q_len, const int* state_slots, float* y,
-                             int is_bf16, int tokens, int segments, int heads, int groups, int d, int p_dim, hipStream_t stream) {
+                             int is_bf16, int tokens, int segments, int heads, int groups, int d, int p_dim, int shorter_than,
+                             hipStream_t stream) {
     if (tokens <= 0 || segments <= 0) return 0;
     if (heads <= 0 || groups <= 0 || heads % groups || d <= 0 || d > 256 || p_dim <= 0 || segments > 65535 ||
         (p_dim + kScanCols - 1) / kScanCols > 65535 || state_stride % 4 || reinterpret_cast<uintptr_t>(state) % 16)
@@ -487,12 +489,294 @@ WLLM_API int wllm_delta_scan(const float* qk, const float* kq, const float* f, c
 #define LAUNCH(T, R)                                                                                                   \
     delta_scan_kernel<T, R><<<grid, kScanThreads, 0, stream>>>(qk, kq, f, beta, static_cast<const T*>(v), state, state_stride, \
                                                                seg_q_start, seg_q_len, state_slots, y, tokens, heads, groups, dp, \
-                                                               p_dim)
+                                                               p_dim, shorter_than)
 #define LAUNCH_R(T)                    \
     if (dp <= 64) LAUNCH(T, 1);        \
     else if (dp <= 128) LAUNCH(T, 2);  \
     else if (dp <= 192) LAUNCH(T, 3);  \
     else LAUNCH(T, 4);
+    if (is_bf16) { LAUNCH_R(bf16) } else { LAUNCH_R(float) }
+#undef LAUNCH_R
+#undef LAUNCH
+    return launch_status();
+}
+
+// ---- the same recurrence over many tokens, 16 at a time on the matrix cores.  With D_t the product of the decays of a
+// chunk's tokens up to t (a number a channel), and every product of decays between two tokens formed from the decays
+// between them (never as a quotient), the 16 tokens' writes are the solution of a triangular system:
+//   W = V - (D K) S0;   U = M W;   O = (D Q) S0 + N W;   S = D_16 S0 + Kh^T U
+// with (D K)_t = D_t k_t, (D Q)_t = D_t q_t, Kh_s = k_s times the decays behind s,
+//   A_ts = k_t . (decays s < r <= t) k_s,   B_ts = q_t . (decays s < r <= t) k_s (s <= t),
+//   M = (I + diag(beta) strictly_lower(A))^-1 diag(beta),   N = B M
+// none of which depends on the memory: `delta_chunk_kernel` makes them for all chunks and heads at once, and
+// `delta_chunk_scan_kernel` walks a segment's chunks in order with v_mfma_f32_16x16x4_f32 (float32 in and out).  A chunk
+// begins every 16 tokens of a segment; the last one is filled with tokens that change nothing (k = q = 0, f = 1, beta = 0).
+// Chunk c of segment s lies at place q_start / 16 + s + c of the scratch (no two chunks share one), its operands of head h
+// as [16][C] D K, [16][C] D Q, [C][16] Kh, [C] D_16, [16][16] M, [16][16] N with C = the channels padded to a multiple of 64.
+constexpr int kChunk = 16;
+
+__host__ __device__ __forceinline__ size_t chunk_floats(int c) { return static_cast<size_t>(3 * kChunk + 1) * c + 2 * kChunk * kChunk; }
+
+template <int R>        // C = 64 R
+__global__ void __launch_bounds__(256)
+delta_chunk_kernel(const float* __restrict__ qk, const float* __restrict__ f, const float* __restrict__ beta,
+                   const int* __restrict__ token_segment, const int* __restrict__ seg_q_start, const int* __restrict__ seg_q_len,
+                   float* __restrict__ chunks, int tokens, int heads, int groups, int dp, int from) {
+    constexpr int C = 64 * R;
+    __shared__ __align__(16) float k_s[kChunk * C], q_s[kChunk * C], f_s[kChunk * C];
+    __shared__ float a_s[kChunk][kChunk + 1], b_s[kChunk][kChunk + 1], m_s[kChunk][kChunk + 1];
+    __shared__ float beta_s[kChunk];
+    const int h = blockIdx.y, g = h / (heads / groups);
+    const int tid = threadIdx.x, lane = tid % kWave, wave = tid / kWave;
+    // which of these 16 tokens begins a chunk (at most two do: a segment that is walked in chunks has 16 tokens or more)
+    bool begins = false;
+    {
+        const int token = blockIdx.x * kChunk + lane;
+        if (lane < kChunk && token < tokens) {
+            const int seg = token_segment[token];
+            begins = seg_q_len[seg] >= from && (token - seg_q_start[seg]) % kChunk == 0;
+        }
+    }
+    unsigned long long starts = __ballot(begins);
+    while (starts) {
+        const int token = blockIdx.x * kChunk + __ffsll(starts) - 1;
+        starts &= starts - 1;
+        const int seg = token_segment[token], q_start = seg_q_start[seg];
+        const int local = token - q_start, count = min(kChunk, seg_q_len[seg] - local);
+        const size_t place = static_cast<size_t>(q_start / kChunk + seg + local / kChunk);
+        float* out = chunks + (place * heads + h) * chunk_floats(C);
+        const size_t q_width = static_cast<size_t>(groups) * dp, f_width = static_cast<size_t>(heads) * dp;
+        __syncthreads();                          // the chunk before is read out
+        for (int four = tid; four < kChunk * C / 4; four += 256) {
+            const int t = four / (C / 4), i = four % (C / 4) * 4;
+            float4 k = make_float4(0.f, 0.f, 0.f, 0.f), q = k, d = make_float4(1.f, 1.f, 1.f, 1.f);
+            if (t < count && i < dp) {
+                const float* at = qk + static_cast<size_t>(token + t) * q_width + static_cast<size_t>(g) * dp + i;
+                q = *reinterpret_cast<const float4*>(at);
+                k = *reinterpret_cast<const float4*>(at + static_cast<size_t>(tokens) * q_width);
+                d = *reinterpret_cast<const float4*>(f + static_cast<size_t>(token + t) * f_width + static_cast<size_t>(h) * dp + i);
+            }
+            reinterpret_cast<float4*>(k_s)[four] = k;
+            reinterpret_cast<float4*>(q_s)[four] = q;
+            reinterpret_cast<float4*>(f_s)[four] = d;
+        }
+        if (tid < kChunk) beta_s[tid] = tid < count ? beta[static_cast<size_t>(token + tid) * heads + h] : 0.f;
+        __syncthreads();
+        // A and B: 16 lanes hold the key of token s, which decays as t goes on
+        {
+            const int s = tid / kChunk, sl = tid % kChunk;
+            float4 r[R];
+#pragma unroll
+            for (int j = 0; j < R; ++j) r[j] = *reinterpret_cast<const float4*>(k_s + s * C + 64 * j + 4 * sl);
+            const int first = wave * (kWave / kChunk);            // the wavefront's first s
+            for (int t = 0; t < kChunk; ++t) {
+                float a = 0.f, b = 0.f;
+                if (t >= first) {
+#pragma unroll
+                    for (int j = 0; j < R; ++j) {
+                        const int at = t * C + 64 * j + 4 * sl;
+                        const float4 kt = *reinterpret_cast<const float4*>(k_s + at), qt = *reinterpret_cast<const float4*>(q_s + at);
+                        if (t > s) {
+                            const float4 ft = *reinterpret_cast<const float4*>(f_s + at);
+                            r[j].x *= ft.x;
+                            r[j].y *= ft.y;
+                            r[j].z *= ft.z;
+                            r[j].w *= ft.w;
+                        }
+                        a += dot4(r[j], kt);
+                        b += dot4(r[j], qt);
+                    }
+                    a = row_sum(a);
+                    b = row_sum(b);
+                }
+                if (sl == 0) {
+                    a_s[t][s] = t > s ? a : 0.f;
+                    b_s[t][s] = t >= s ? b : 0.f;
+                }
+            }
+        }
+        // the decays up to and behind every token, a channel a thread
+        for (int c = tid; c < C; c += 256) {
+            float decay = 1.f;
+#pragma unroll
+            for (int t = 0; t < kChunk; ++t) {
+                decay *= f_s[t * C + c];
+                out[t * C + c] = k_s[t * C + c] * decay;
+                out[(kChunk + t) * C + c] = q_s[t * C + c] * decay;
+            }
+            out[3 * kChunk * C + c] = decay;
+            float kh[kChunk], behind = 1.f;
+#pragma unroll
+            for (int t = kChunk - 1; t >= 0; --t) {
+                kh[t] = k_s[t * C + c] * behind;
+                behind *= f_s[t * C + c];
+            }
+#pragma unroll
+            for (int t = 0; t < kChunk; t += 4)
+                *reinterpret_cast<float4*>(out + 2 * kChunk * C + c * kChunk + t) = make_float4(kh[t], kh[t + 1], kh[t + 2], kh[t + 3]);
+        }
+        __syncthreads();
+        float* mn = out + (3 * kChunk + 1) * C;
+        if (tid < kChunk) {
+            // a column of M: m_t = beta_t (delta_tj - sum over s < t of A_ts m_s)
+            float m[kChunk];
+#pragma unroll
+            for (int t = 0; t < kChunk; ++t) {
+                float sum = 0.f;
+#pragma unroll
+                for (int s = 0; s < t; ++s) sum = fmaf(a_s[t][s], m[s], sum);
+                m[t] = beta_s[t] * ((t == tid ? 1.f : 0.f) - sum);
+                m_s[t][tid] = m[t];
+            }
+        }
+        __syncthreads();
+        {
+            const int t = tid / kChunk, j = tid % kChunk;
+            float n = 0.f;
+#pragma unroll
+            for (int s = 0; s < kChunk; ++s) n = fmaf(b_s[t][s], m_s[s][j], n);
+            mn[tid] = m_s[t][j];
+            mn[kChunk * kChunk + tid] = n;
+        }
+    }
+}
+
+// A workgroup owns (head, segment, 16 value columns).  The channels are cut over its four wavefronts, each with TILES tiles
+// of 16 of them: lane (i, g) holds the memory's channels 4g .. 4g + 3 of a tile in column i, which is what the product
+// leaves and, channel by channel, what it takes (the k-th of four products takes the channels 4g + k), so the memory never
+// moves between lanes.  The wavefronts' parts of (D K) S0 and (D Q) S0 meet in shared memory (two places in turn: one
+// barrier a chunk); what follows every wavefront makes for itself.  The next chunk's operands are asked for first.
+typedef float delta_float4 __attribute__((ext_vector_type(4)));
+
+template <typename T, int TILES>
+__global__ void __launch_bounds__(256)
+delta_chunk_scan_kernel(const float* __restrict__ chunks, const T* __restrict__ v, float* __restrict__ state,
+                        long long state_stride, const int* __restrict__ seg_q_start, const int* __restrict__ seg_q_len,
+                        const int* __restrict__ state_slots, float* __restrict__ y, int heads, int dp, int p_dim, int from) {
+    constexpr int C = 64 * TILES;
+    __shared__ delta_float4 part_s[2][4][2][kWave];
+    const int h = blockIdx.x, seg = blockIdx.y, p0 = blockIdx.z * 16;
+    const int q_len = seg_q_len[seg], q_start = seg_q_start[seg];
+    if (q_len < from) return;
+    const int lane = threadIdx.x % kWave, wave = threadIdx.x / kWave;
+    const int i = lane % 16, g = lane / 16;
+    const int p = p0 + i;
+    const bool live = p < p_dim;
+    float* s_col = state + static_cast<size_t>(state_slots[seg]) * state_stride + (static_cast<size_t>(h) * p_dim + p) * dp;
+    const int ch0 = wave * 16 * TILES;
+    delta_float4 s[TILES];
+#pragma unroll
+    for (int j = 0; j < TILES; ++j) {
+        const int ch = ch0 + 16 * j + 4 * g;
+        s[j] = live && ch < dp ? *reinterpret_cast<const delta_float4*>(s_col + ch) : delta_float4{0.f, 0.f, 0.f, 0.f};
+    }
+    struct Operands {
+        delta_float4 k[TILES], q[TILES], kh[TILES], d[TILES], m, n;
+        float v[4];
+    };
+    const float* base = chunks + (static_cast<size_t>(q_start / kChunk + seg) * heads + h) * chunk_floats(C);
+    const T* v_col = v + static_cast<size_t>(q_start) * heads * p_dim + static_cast<size_t>(h) * p_dim + p;
+    auto load = [&](int c) {
+        Operands o;
+        const float* at = base + static_cast<size_t>(c) * heads * chunk_floats(C);
+#pragma unroll
+        for (int j = 0; j < TILES; ++j) {
+            const int ch = ch0 + 16 * j;
+            o.k[j] = *reinterpret_cast<const delta_float4*>(at + i * C + ch + 4 * g);
+            o.q[j] = *reinterpret_cast<const delta_float4*>(at + (kChunk + i) * C + ch + 4 * g);
+            o.kh[j] = *reinterpret_cast<const delta_float4*>(at + 2 * kChunk * C + (ch + i) * kChunk + 4 * g);
+            o.d[j] = *reinterpret_cast<const delta_float4*>(at + 3 * kChunk * C + ch + 4 * g);
+        }
+        const float* mn = at + (3 * kChunk + 1) * C;
+        o.m = *reinterpret_cast<const delta_float4*>(mn + i * kChunk + 4 * g);
+        o.n = *reinterpret_cast<const delta_float4*>(mn + kChunk * kChunk + i * kChunk + 4 * g);
+#pragma unroll
+        for (int u = 0; u < 4; ++u) {
+            const int t = c * kChunk + 4 * g + u;
+            o.v[u] = live && t < q_len ? to_float(v_col[static_cast<size_t>(t) * heads * p_dim]) : 0.f;
+        }
+        return o;
+    };
+    const int count = (q_len + kChunk - 1) / kChunk;
+    Operands now = load(0);
+    for (int c = 0; c < count; ++c) {
+        const Operands next = load(min(c + 1, count - 1));
+        delta_float4 seen = {0.f, 0.f, 0.f, 0.f}, read = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int j = 0; j < TILES; ++j)
+#pragma unroll
+            for (int u = 0; u < 4; ++u) {
+                seen = __builtin_amdgcn_mfma_f32_16x16x4f32(now.k[j][u], s[j][u], seen, 0, 0, 0);
+                read = __builtin_amdgcn_mfma_f32_16x16x4f32(now.q[j][u], s[j][u], read, 0, 0, 0);
+            }
+        part_s[c % 2][wave][0][lane] = seen;
+        part_s[c % 2][wave][1][lane] = read;
+        // the memory decays while the parts meet
+#pragma unroll
+        for (int j = 0; j < TILES; ++j) s[j] *= now.d[j];
+        __syncthreads();
+        seen = part_s[c % 2][0][0][lane];
+        read = part_s[c % 2][0][1][lane];
+#pragma unroll
+        for (int w = 1; w < 4; ++w) {
+            seen += part_s[c % 2][w][0][lane];
+            read += part_s[c % 2][w][1][lane];
+        }
+        delta_float4 u4 = {0.f, 0.f, 0.f, 0.f}, left;
+#pragma unroll
+        for (int u = 0; u < 4; ++u) left[u] = now.v[u] - seen[u];
+#pragma unroll
+        for (int u = 0; u < 4; ++u) u4 = __builtin_amdgcn_mfma_f32_16x16x4f32(now.m[u], left[u], u4, 0, 0, 0);
+#pragma unroll
+        for (int u = 0; u < 4; ++u)
+#pragma unroll
+            for (int j = 0; j < TILES; ++j) s[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(now.kh[j][u], u4[u], s[j], 0, 0, 0);
+#pragma unroll
+        for (int u = 0; u < 4; ++u) read = __builtin_amdgcn_mfma_f32_16x16x4f32(now.n[u], left[u], read, 0, 0, 0);
+        // wavefront w writes the tokens 4g + w
+        const int t = c * kChunk + 4 * g + wave;
+        const float o = wave == 0 ? read[0] : wave == 1 ? read[1] : wave == 2 ? read[2] : read[3];
+        if (live && t < q_len) y[static_cast<size_t>(q_start + t) * heads * p_dim + static_cast<size_t>(h) * p_dim + p] = o;
+        now = next;
+    }
+    if (live) {
+#pragma unroll
+        for (int j = 0; j < TILES; ++j) {
+            const int ch = ch0 + 16 * j + 4 * g;
+            if (ch < dp) *reinterpret_cast<delta_float4*>(s_col + ch) = s[j];
+        }
+    }
+}
+
+// Floats of the scratch for a step of `tokens` tokens in `segments` segments.
+WLLM_API long long wllm_delta_chunk_floats(int tokens, int segments, int heads, int d) {
+    const int c = (d + 63) / 64 * 64;
+    return static_cast<long long>(tokens / kChunk + segments + 1) * heads * static_cast<long long>(chunk_floats(c));
+}
+
+// Segments of `from` tokens (16 at least) and more; the others are left alone.
+WLLM_API int wllm_delta_chunk_scan(const float* qk, const float* f, const float* beta, const void* v, float* state,
+                                   long long state_stride, const int* token_segment, const int* seg_q_start, const int* seg_q_len,
+                                   const int* state_slots, float* y, float* chunks, int is_bf16, int tokens, int segments, int heads,
+                                   int groups, int d, int p_dim, int from, hipStream_t stream) {
+    if (tokens <= 0 || segments <= 0) return 0;
+    if (heads <= 0 || heads > 65535 || groups <= 0 || heads % groups || d <= 0 || d > 256 || p_dim <= 0 || segments > 65535 ||
+        (p_dim + 15) / 16 > 65535 || from < kChunk || state_stride % 4 || reinterpret_cast<uintptr_t>(state) % 16 ||
+        reinterpret_cast<uintptr_t>(chunks) % 16)
+        return -1;
+    const int dp = (d + 3) / 4 * 4, r = (d + 63) / 64;
+    const dim3 chunk_grid((tokens + kChunk - 1) / kChunk, heads), grid(heads, segments, (p_dim + 15) / 16);
+#define LAUNCH(T, R)                                                                                                   \
+    delta_chunk_kernel<R><<<chunk_grid, 256, 0, stream>>>(qk, f, beta, token_segment, seg_q_start, seg_q_len, chunks, tokens,  \
+                                                          heads, groups, dp, from);                                     \
+    if (const int err = launch_status()) return err;                                                                   \
+    delta_chunk_scan_kernel<T, R><<<grid, 256, 0, stream>>>(chunks, static_cast<const T*>(v), state, state_stride, seg_q_start, \
+                                                            seg_q_len, state_slots, y, heads, dp, p_dim, from)
+#define LAUNCH_R(T)                     \
+    if (r == 1) { LAUNCH(T, 1); }       \
+    else if (r == 2) { LAUNCH(T, 2); }  \
+    else if (r == 3) { LAUNCH(T, 3); }  \
+    else { LAUNCH(T, 4); }
     if (is_bf16) { LAUNCH_R(bf16) } else { LAUNCH_R(float) }
 #undef LAUNCH_R
 #undef LAUNCH

@@ -1241,12 +1241,12 @@ def delta_inputs(xqkv: torch.Tensor, z: torch.Tensor, b: torch.Tensor, conv_weig
 
 def delta_scan(qk: torch.Tensor, kq: torch.Tensor, f: torch.Tensor, beta: torch.Tensor, v: torch.Tensor, state: torch.Tensor,
                seg_q_start: torch.Tensor, seg_q_len: torch.Tensor, state_slots: torch.Tensor, y: torch.Tensor, *, heads: int,
-               groups: int, head_dim: int, value_dim: int) -> None:
+               groups: int, head_dim: int, value_dim: int, shorter_than: Optional[int] = None) -> None:
     """The delta rule over each segment's tokens in order, from and into the request's carried memory.  Per head h (group
     h // (heads // groups) of q and k):  S = diag(f) S;  u = beta (v - S^T k);  S += k u^T;  y = S^T q, the last computed as
     (diag(f) S)^T q + u (k . q).  Operands as `delta_inputs` leaves them; state float32 [slots, W] (W a multiple of four),
     whose row state_slots[segment] begins with [heads, P, DP]: a head's memory, a value column after the other;
-    y float32 [n, heads * P].  All float32."""
+    y float32 [n, heads * P].  All float32.  `shorter_than`: segments of that many tokens and more are left alone."""
     _delta_sizes(heads, groups, head_dim, value_dim)
     dp = delta_padded(head_dim)
     _need(v.dim() == 2 and v.dtype in _ACT, "v: expected T [n, heads * value_dim]")
@@ -1262,7 +1262,47 @@ def delta_scan(qk: torch.Tensor, kq: torch.Tensor, f: torch.Tensor, beta: torch.
     _segments(seg_q_start, seg_q_len, state_slots)
     _dense(y, "y", torch.float32, (n, heads * value_dim))
     if n:
-        call("delta_scan", qk, kq, f, beta, v, state, seg_q_start, seg_q_len, state_slots, y, heads, groups, head_dim, value_dim)
+        call("delta_scan", qk, kq, f, beta, v, state, seg_q_start, seg_q_len, state_slots, y, heads, groups, head_dim, value_dim,
+             **({"shorter_than": int(shorter_than)} if shorter_than is not None else {}))
+
+
+DELTA_CHUNK = 16        # tokens a chunk of `delta_chunk_scan`
+
+
+def delta_chunk_size(tokens: int, segments: int, heads: int, head_dim: int) -> int:
+    """Floats of the scratch `delta_chunk_scan` needs for a step: a place for every chunk of every segment."""
+    c = -(-head_dim // 64) * 64
+    return (tokens // DELTA_CHUNK + segments + 1) * heads * ((3 * DELTA_CHUNK + 1) * c + 2 * DELTA_CHUNK * DELTA_CHUNK)
+
+
+def delta_chunk_scan(qk: torch.Tensor, f: torch.Tensor, beta: torch.Tensor, v: torch.Tensor, state: torch.Tensor,
+                     token_segment: torch.Tensor, seg_q_start: torch.Tensor, seg_q_len: torch.Tensor, state_slots: torch.Tensor,
+                     y: torch.Tensor, chunks: torch.Tensor, *, heads: int, groups: int, head_dim: int, value_dim: int,
+                     from_tokens: int) -> None:
+    """What `delta_scan` does, for the segments of `from_tokens` tokens (at least `DELTA_CHUNK`) and more; the others are left
+    alone.  The tokens are taken in chunks of 16 from the segment's start, a chunk's writes as the solution of a triangular
+    system, its products on the matrix cores, all in float32: the same numbers up to the order of sums.  `chunks`: float32
+    scratch of `delta_chunk_size` elements; the other operands as in `delta_scan`."""
+    _delta_sizes(heads, groups, head_dim, value_dim)
+    dp = delta_padded(head_dim)
+    _need(v.dim() == 2 and v.dtype in _ACT, "v: expected T [n, heads * value_dim]")
+    n = v.shape[0]
+    _dense(v, "v", _ACT, (n, heads * value_dim))
+    _dense(qk, "qk", torch.float32, (2, n, groups * dp))
+    _dense(f, "f", torch.float32, (n, heads * dp))
+    _dense(beta, "beta", torch.float32, (n, heads))
+    _dense(state, "state", torch.float32)
+    _need(state.dim() == 2 and state.shape[1] >= delta_state_size(heads, head_dim, value_dim) and state.shape[1] % 4 == 0,
+          "state: a row begins with [heads, P, DP] and is a multiple of four floats")
+    _dense(token_segment, "token_segment", torch.int32, (n,))
+    s = _segments(seg_q_start, seg_q_len, state_slots)
+    _dense(y, "y", torch.float32, (n, heads * value_dim))
+    _need(from_tokens >= DELTA_CHUNK, f"from_tokens: at least {DELTA_CHUNK}")
+    _dense(chunks, "chunks", torch.float32)
+    _need(chunks.numel() >= delta_chunk_size(n, s, heads, head_dim), "chunks: smaller than delta_chunk_size")
+    if n:
+        call("delta_chunk_scan", qk, f, beta, v, state, token_segment, seg_q_start, seg_q_len, state_slots, y, chunks, heads, groups,
+             head_dim, value_dim, int(from_tokens))
 
 
 # ---- a mixture of experts ------------------------------------------------------------------------------
@@ -1614,11 +1654,18 @@ def _register_own() -> None:
                     p(v), p(f), p(beta), q_scale, unit_eps, bf(xqkv), xqkv.shape[0], seg_q_start.shape[0], heads, groups, head_dim,
                     value_dim, conv_weight.shape[0], int(single_tokens), stream))
     register_op("delta_scan", entry_point="wllm_delta_scan",
-                argtypes=[c_void_p] * 6 + [c_longlong] + [c_void_p] * 4 + [c_int] * 7 + [c_void_p],
+                argtypes=[c_void_p] * 6 + [c_longlong] + [c_void_p] * 4 + [c_int] * 8 + [c_void_p],
                 launch=lambda fn, stream, qk, kq, f, beta, v, state, seg_q_start, seg_q_len, state_slots, y, heads, groups, head_dim,
-                value_dim: fn(
+                value_dim, shorter_than=0x7fffffff: fn(
                     p(qk), p(kq), p(f), p(beta), p(v), p(state), state.stride(0), p(seg_q_start), p(seg_q_len), p(state_slots), p(y),
-                    bf(v), v.shape[0], seg_q_start.shape[0], heads, groups, head_dim, value_dim, stream))
+                    bf(v), v.shape[0], seg_q_start.shape[0], heads, groups, head_dim, value_dim, shorter_than, stream))
+    register_op("delta_chunk_scan", entry_point="wllm_delta_chunk_scan",
+                argtypes=[c_void_p] * 5 + [c_longlong] + [c_void_p] * 6 + [c_int] * 8 + [c_void_p],
+                launch=lambda fn, stream, qk, f, beta, v, state, token_segment, seg_q_start, seg_q_len, state_slots, y, chunks, heads,
+                groups, head_dim, value_dim, from_tokens: fn(
+                    p(qk), p(f), p(beta), p(v), p(state), state.stride(0), p(token_segment), p(seg_q_start), p(seg_q_len),
+                    p(state_slots), p(y), p(chunks), bf(v), v.shape[0], seg_q_start.shape[0], heads, groups, head_dim, value_dim,
+                    from_tokens, stream))
     register_op("moe_route", entry_point="wllm_moe_route",
                 argtypes=[c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int,
                           c_int, c_int, c_float, c_int, c_int, c_void_p],

@@ -15,7 +15,8 @@ A request carries S and the convolutions' last taps - 1 inputs from step to step
 cache manager (`ops.delta_state_size` floats, a value column after the other, then [taps - 1, channels]; zeroed at
 admission, which is both the zero memory and the zeros before a sequence's start).  The kernels walk every segment's
 tokens in order from that row and leave it for the next step, so a prompt may be cut anywhere, and a decoded token
-is a segment of one.  Everything the kernels read of the step lies in device arrays, so a decode step can be
+is a segment of one.  Two kernels do so: token by token, or, for the portions of a step that are long enough, chunk by
+chunk of 16 tokens on the matrix cores (the same numbers up to the order of float32 sums).  Everything the kernels read of the step lies in device arrays, so a decode step can be
 captured in a graph.
 """
 from __future__ import annotations
@@ -29,6 +30,9 @@ from wllm_amd.parts.common import Product, load_matrix
 from wllm_amd.parts.registry import register_mixer
 from wllm_amd.parts.specs import DeltaRuleSpec
 from wllm_amd.weights.checkpoint import ExpectedTensor, WeightError
+
+
+LONG_PORTION = 32       # tokens of a request in a step from which its recurrence is walked in chunks
 
 
 @register_mixer("delta_rule")
@@ -143,7 +147,13 @@ class DeltaRuleMixer:
                          self.memory_size, ctx.token_segment, *segments, qk, kq, v, f, beta, q_scale=s.q_scale,
                          unit_eps=s.unit_eps, single_tokens=ctx.max_q_len == 1 and ctx.num_segments == n, **sizes)
         y = ctx.buffer("delta_y", (n, self.v_width), f32)
-        ops.delta_scan(qk, kq, f, beta, v, state, *segments, y, **sizes)
+        # long portions go 16 tokens at a time over the matrix cores, the others (decoded tokens) token by token
+        long = ctx.max_q_len >= LONG_PORTION
+        if long:
+            chunks = ctx.buffer("delta_chunks", (ops.delta_chunk_size(n, ctx.num_segments, s.num_heads, s.head_dim),), f32)
+            ops.delta_chunk_scan(qk, f, beta, v, state, ctx.token_segment, *segments, y, chunks, from_tokens=LONG_PORTION, **sizes)
+        if not long or int(ctx.host_q_len.min()) < LONG_PORTION:
+            ops.delta_scan(qk, kq, f, beta, v, state, *segments, y, shorter_than=LONG_PORTION if long else None, **sizes)
         out = product_input if product_input is not None else ctx.buffer("delta_out", (n, self.v_width), h.dtype)
         ops.head_norm_gate(y, outer[:, self.outer:self.outer + self.v_width], self.norm_w, out, heads=s.num_heads,
                            eps=s.norm_eps, activation="sigmoid")
