@@ -648,9 +648,10 @@ delta_chunk_kernel(const float* __restrict__ qk, const float* __restrict__ f, co
 // barrier a chunk); what follows every wavefront makes for itself.  The next chunk's operands are asked for first.
 typedef float delta_float4 __attribute__((ext_vector_type(4)));
 
+// (two workgroups a compute unit at least: the products then keep their sums in the registers the rest is in)
 template <typename T, int TILES>
-__global__ void __launch_bounds__(256)
-delta_chunk_scan_kernel(const float* __restrict__ chunks, const T* __restrict__ v, float* __restrict__ state,
+__global__ void __launch_bounds__(256, 2)
+delta_chunk_scan_kernel(const float* chunks, const T* v, float* __restrict__ state,
                         long long state_stride, const int* __restrict__ seg_q_start, const int* __restrict__ seg_q_len,
                         const int* __restrict__ state_slots, float* __restrict__ y, int heads, int dp, int p_dim, int from) {
     constexpr int C = 64 * TILES;
@@ -672,35 +673,39 @@ delta_chunk_scan_kernel(const float* __restrict__ chunks, const T* __restrict__ 
     }
     struct Operands {
         delta_float4 k[TILES], q[TILES], kh[TILES], d[TILES], m, n;
-        float v[4];
+        T v[4];
     };
     const float* base = chunks + (static_cast<size_t>(q_start / kChunk + seg) * heads + h) * chunk_floats(C);
-    const T* v_col = v + static_cast<size_t>(q_start) * heads * p_dim + static_cast<size_t>(h) * p_dim + p;
+    // where this lane's operands lie in a chunk's (unsigned: a lane's offset beside an address that is the same in all lanes)
+    const unsigned k_at = i * C + ch0 + 4 * g, kh_at = 2 * kChunk * C + (ch0 + i) * kChunk + 4 * g, d_at = 3 * kChunk * C + ch0 + 4 * g;
+    const unsigned m_at = (3 * kChunk + 1) * C + i * kChunk + 4 * g;
+    const unsigned v_row = static_cast<unsigned>(heads) * p_dim, v_at = static_cast<unsigned>(min(p, p_dim - 1));
+    const T* v_first = v + static_cast<size_t>(q_start) * v_row + static_cast<size_t>(h) * p_dim;
+    float* y_first = y + static_cast<size_t>(q_start) * v_row + static_cast<size_t>(h) * p_dim;
     auto load = [&](int c) {
         Operands o;
         const float* at = base + static_cast<size_t>(c) * heads * chunk_floats(C);
 #pragma unroll
         for (int j = 0; j < TILES; ++j) {
-            const int ch = ch0 + 16 * j;
-            o.k[j] = *reinterpret_cast<const delta_float4*>(at + i * C + ch + 4 * g);
-            o.q[j] = *reinterpret_cast<const delta_float4*>(at + (kChunk + i) * C + ch + 4 * g);
-            o.kh[j] = *reinterpret_cast<const delta_float4*>(at + 2 * kChunk * C + (ch + i) * kChunk + 4 * g);
-            o.d[j] = *reinterpret_cast<const delta_float4*>(at + 3 * kChunk * C + ch + 4 * g);
+            o.k[j] = *reinterpret_cast<const delta_float4*>(at + k_at + 16 * j);
+            o.q[j] = *reinterpret_cast<const delta_float4*>(at + k_at + kChunk * C + 16 * j);
+            o.kh[j] = *reinterpret_cast<const delta_float4*>(at + kh_at + 16 * kChunk * j);
+            o.d[j] = *reinterpret_cast<const delta_float4*>(at + d_at + 16 * j);
         }
-        const float* mn = at + (3 * kChunk + 1) * C;
-        o.m = *reinterpret_cast<const delta_float4*>(mn + i * kChunk + 4 * g);
-        o.n = *reinterpret_cast<const delta_float4*>(mn + kChunk * kChunk + i * kChunk + 4 * g);
+        o.m = *reinterpret_cast<const delta_float4*>(at + m_at);
+        o.n = *reinterpret_cast<const delta_float4*>(at + m_at + kChunk * kChunk);
+        const T* v_chunk = v_first + static_cast<size_t>(c) * kChunk * v_row;
+        const unsigned beyond = min(kChunk, q_len - c * kChunk) - 1;          // the chunk's last token
 #pragma unroll
         for (int u = 0; u < 4; ++u) {
-            const int t = c * kChunk + 4 * g + u;
-            o.v[u] = live && t < q_len ? to_float(v_col[static_cast<size_t>(t) * heads * p_dim]) : 0.f;
+            // (beyond the segment's last token, that token's once more: what it is multiplied by is zero.  Nothing is made of
+            // the values here, and no branch stands before the loads: they are not waited for)
+            o.v[u] = v_chunk[min(static_cast<unsigned>(4 * g + u), beyond) * v_row + v_at];
         }
         return o;
     };
     const int count = (q_len + kChunk - 1) / kChunk;
-    Operands now = load(0);
-    for (int c = 0; c < count; ++c) {
-        const Operands next = load(min(c + 1, count - 1));
+    auto walk = [&](int c, const Operands& now) {
         delta_float4 seen = {0.f, 0.f, 0.f, 0.f}, read = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
         for (int j = 0; j < TILES; ++j)
@@ -714,7 +719,10 @@ delta_chunk_scan_kernel(const float* __restrict__ chunks, const T* __restrict__ 
         // the memory decays while the parts meet
 #pragma unroll
         for (int j = 0; j < TILES; ++j) s[j] *= now.d[j];
-        __syncthreads();
+        // (a barrier for what lies in shared memory alone: the operands of the chunks ahead stay on their way)
+        asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+        __builtin_amdgcn_s_barrier();
+        asm volatile("" ::: "memory");
         seen = part_s[c % 2][0][0][lane];
         read = part_s[c % 2][0][1][lane];
 #pragma unroll
@@ -724,7 +732,7 @@ delta_chunk_scan_kernel(const float* __restrict__ chunks, const T* __restrict__ 
         }
         delta_float4 u4 = {0.f, 0.f, 0.f, 0.f}, left;
 #pragma unroll
-        for (int u = 0; u < 4; ++u) left[u] = now.v[u] - seen[u];
+        for (int u = 0; u < 4; ++u) left[u] = (c * kChunk + 4 * g + u < q_len ? to_float(now.v[u]) : 0.f) - seen[u];
 #pragma unroll
         for (int u = 0; u < 4; ++u) u4 = __builtin_amdgcn_mfma_f32_16x16x4f32(now.m[u], left[u], u4, 0, 0, 0);
 #pragma unroll
@@ -734,11 +742,24 @@ delta_chunk_scan_kernel(const float* __restrict__ chunks, const T* __restrict__ 
 #pragma unroll
         for (int u = 0; u < 4; ++u) read = __builtin_amdgcn_mfma_f32_16x16x4f32(now.n[u], left[u], read, 0, 0, 0);
         // wavefront w writes the tokens 4g + w
-        const int t = c * kChunk + 4 * g + wave;
+        const int t = 4 * g + wave;
         const float o = wave == 0 ? read[0] : wave == 1 ? read[1] : wave == 2 ? read[2] : read[3];
-        if (live && t < q_len) y[static_cast<size_t>(q_start + t) * heads * p_dim + static_cast<size_t>(h) * p_dim + p] = o;
-        now = next;
+        if (live && c * kChunk + t < q_len) (y_first + static_cast<size_t>(c) * kChunk * v_row)[t * v_row + v_at] = o;
+    };
+    // two chunks' operands in turn, each asked for while the chunk before is walked (beyond the last: the last's once more)
+    Operands a = load(0);
+    int c = 0;
+    for (; c + 1 < count; c += 2) {
+        // (the loads stay where they are written: `chunks` and `v` may alias as far as the compiler knows, and the empty
+        // statements touch memory)
+        const Operands b = load(c + 1);
+        asm volatile("" ::: "memory");
+        walk(c, a);
+        a = load(min(c + 2, count - 1));
+        asm volatile("" ::: "memory");
+        walk(c + 1, b);
     }
+    if (c < count) walk(c, a);
     if (live) {
 #pragma unroll
         for (int j = 0; j < TILES; ++j) {
