@@ -180,6 +180,236 @@ norm_add_kernel(float* __restrict__ x, const TD* __restrict__ delta, int splits,
     }
 }
 
+// The same for rows of a multiple of four elements, held in registers: a thread keeps G groups of four consecutive
+// elements and moves 16 (bfloat16: 8) bytes at a time; everything a row needs is asked for before the first sum.
+// CONV: the launch also convolves (`conv_aligned`: the carried rows begin at multiples of 16 bytes).
+template <typename T> struct alignas(4 * sizeof(T)) NormFour { T v[4]; };
+
+// Mean and 1 / sqrt(variance + eps) (a norm of kind RMS: mean 0) of the row that the workgroup's threads hold.
+template <int G>
+__device__ __forceinline__ void held_stats(const float (&v)[G][4], int hidden, int kind, float eps, float* scratch, float& mean,
+                                           float& inv) {
+    mean = 0.f;
+    inv = 1.f;
+    if (kind == kNormNone) return;
+    const float count = static_cast<float>(hidden);
+    if (kind == kNormLayer) {
+        float s = 0.f;
+#pragma unroll
+        for (int e = 0; e < G; ++e) s += (v[e][0] + v[e][1]) + (v[e][2] + v[e][3]);       // (zeros beyond the row)
+        mean = block_sum(s, scratch) / count;
+    }
+    float ss = 0.f;
+#pragma unroll
+    for (int e = 0; e < G; ++e) {
+        if (static_cast<int>(threadIdx.x + e * blockDim.x) * 4 < hidden) {
+#pragma unroll
+            for (int u = 0; u < 4; ++u) {
+                const float d = v[e][u] - mean;
+                ss += d * d;
+            }
+        }
+    }
+    inv = 1.f / sqrtf(block_sum(ss, scratch) / count + eps);
+}
+
+template <typename TD, typename TO, int G, bool CONV>
+__global__ void __launch_bounds__(1024)
+norm_add_four_kernel(float* __restrict__ x, const TD* __restrict__ delta, int splits, size_t split_stride, int d_kind,
+                     const float* __restrict__ d_weight, float d_eps, float d_offset, const int* __restrict__ rows,
+                     TO* __restrict__ out, int o_kind, const float* __restrict__ o_weight, float o_eps, float o_offset,
+                     int hidden, NormJoin join, NormConv conv, int conv_aligned) {
+    __shared__ float scratch[16];
+    const int orow = blockIdx.x;
+    const int irow = rows ? rows[orow] : orow;
+    // the carried rows (and taps) of this thread's elements, the first ones asked for before anything else
+    constexpr int kHeldTaps = CONV ? 4 : 1;
+    float* carried = CONV ? conv.state + static_cast<size_t>(conv.state_slots[orow]) * conv.state_stride + conv.carried_offset : nullptr;
+    NormFour<float> held_w[CONV ? G : 1][kHeldTaps], held_c[CONV ? G : 1][kHeldTaps];
+    auto carried_four = [&](int k, int i) {
+        const float* p = carried + static_cast<size_t>(k) * hidden + i;
+        if (conv_aligned) return *reinterpret_cast<const NormFour<float>*>(p);
+        return NormFour<float>{{p[0], p[1], p[2], p[3]}};
+    };
+    auto carry_four = [&](int k, int i, const NormFour<float>& t) {
+        float* p = carried + static_cast<size_t>(k) * hidden + i;
+        if (conv_aligned) {
+            *reinterpret_cast<NormFour<float>*>(p) = t;
+        } else {
+#pragma unroll
+            for (int u = 0; u < 4; ++u) p[u] = t.v[u];
+        }
+    };
+    if (CONV) {
+#pragma unroll
+        for (int e = 0; e < G; ++e) {
+            const int i = static_cast<int>(threadIdx.x + e * blockDim.x) * 4;
+#pragma unroll
+            for (int k = 0; k < kHeldTaps; ++k) {
+                held_w[e][k] = held_c[e][k] = NormFour<float>{{0.f, 0.f, 0.f, 0.f}};
+                if (i < hidden && k < conv.taps)
+                    held_w[e][k] = *reinterpret_cast<const NormFour<float>*>(conv.weight + static_cast<size_t>(k) * hidden + i);
+                if (i < hidden && k + 1 < conv.taps) held_c[e][k] = carried_four(k, i);
+            }
+        }
+    }
+    const size_t base = static_cast<size_t>(irow) * hidden;
+    float xv[G][4], d[G][4], w[G][4];
+    auto at = [&](int e) { return static_cast<int>(threadIdx.x + e * blockDim.x) * 4; };
+    auto weights = [&](const float* from) {
+#pragma unroll
+        for (int e = 0; e < G; ++e) {
+            NormFour<float> t = {{0.f, 0.f, 0.f, 0.f}};
+            if (at(e) < hidden) t = *reinterpret_cast<const NormFour<float>*>(from + at(e));
+#pragma unroll
+            for (int u = 0; u < 4; ++u) w[e][u] = t.v[u];
+        }
+    };
+    // a stack's slices at one place, added in order, several asked for at a time
+    auto stack = [&](const float* from, int count, size_t stride, float (&sum)[4]) {
+        NormFour<float> t = *reinterpret_cast<const NormFour<float>*>(from);
+#pragma unroll
+        for (int u = 0; u < 4; ++u) sum[u] = t.v[u];
+        constexpr int kAhead = 8;
+        for (int s0 = 1; s0 < count; s0 += kAhead) {
+            NormFour<float> q[kAhead];
+#pragma unroll
+            for (int j = 0; j < kAhead; ++j)
+                q[j] = *reinterpret_cast<const NormFour<float>*>(from + static_cast<size_t>(min(s0 + j, count - 1)) * stride);
+#pragma unroll
+            for (int j = 0; j < kAhead; ++j) {
+                if (s0 + j >= count) break;
+#pragma unroll
+                for (int u = 0; u < 4; ++u) sum[u] += q[j].v[u];
+            }
+        }
+    };
+    const float extra_scale = join.extra && join.extra_scale ? join.extra_scale[irow] : 1.f;
+    if (delta && d_kind != kNormNone) weights(d_weight);
+    else if (delta && join.s_kind != kNormNone) weights(join.s_weight);
+    else if (out && o_kind != kNormNone) weights(o_weight);
+#pragma unroll
+    for (int e = 0; e < G; ++e) {
+        const int i = at(e);
+#pragma unroll
+        for (int u = 0; u < 4; ++u) xv[e][u] = d[e][u] = 0.f;
+        if (i >= hidden) continue;
+        const NormFour<float> t = *reinterpret_cast<const NormFour<float>*>(x + base + i);
+#pragma unroll
+        for (int u = 0; u < 4; ++u) xv[e][u] = t.v[u];
+        if (!delta) continue;
+        if (sizeof(TD) == sizeof(float)) {
+            stack(reinterpret_cast<const float*>(delta) + base + i, splits, split_stride, d[e]);
+        } else {
+            const NormFour<TD> q = *reinterpret_cast<const NormFour<TD>*>(delta + base + i);
+#pragma unroll
+            for (int u = 0; u < 4; ++u) d[e][u] = to_float(q.v[u]);
+        }
+        if (join.extra) {
+            float more[4];
+            if (join.extra_bf16) {
+                const NormFour<bf16> q = *reinterpret_cast<const NormFour<bf16>*>(static_cast<const bf16*>(join.extra) + base + i);
+#pragma unroll
+                for (int u = 0; u < 4; ++u) more[u] = to_float(q.v[u]);
+            } else {
+                stack(static_cast<const float*>(join.extra) + base + i, join.extra_splits, join.extra_stride, more);
+            }
+#pragma unroll
+            for (int u = 0; u < 4; ++u) d[e][u] = fmaf(extra_scale, more[u], d[e][u]);
+        }
+    }
+    float mean, inv;
+    if (delta) {
+        if (d_kind != kNormNone) {
+            held_stats<G>(d, hidden, d_kind, d_eps, scratch, mean, inv);
+#pragma unroll
+            for (int e = 0; e < G; ++e)
+#pragma unroll
+                for (int u = 0; u < 4; ++u) d[e][u] = (d[e][u] - mean) * inv * (d_offset + w[e][u]);
+            if (join.s_kind != kNormNone) weights(join.s_weight);
+            else if (out && o_kind != kNormNone) weights(o_weight);
+        }
+#pragma unroll
+        for (int e = 0; e < G; ++e)
+#pragma unroll
+            for (int u = 0; u < 4; ++u) xv[e][u] = at(e) < hidden ? fmaf(join.scale, xv[e][u], d[e][u]) : 0.f;
+        if (join.s_kind != kNormNone) {
+            held_stats<G>(xv, hidden, join.s_kind, join.s_eps, scratch, mean, inv);
+#pragma unroll
+            for (int e = 0; e < G; ++e)
+#pragma unroll
+                for (int u = 0; u < 4; ++u)
+                    xv[e][u] = at(e) < hidden ? (xv[e][u] - mean) * inv * (join.s_offset + w[e][u]) : 0.f;
+            if (out && o_kind != kNormNone) weights(o_weight);
+        } else if (d_kind == kNormNone && out && o_kind != kNormNone) {
+            weights(o_weight);
+        }
+        if (!rows) {
+#pragma unroll
+            for (int e = 0; e < G; ++e) {
+                if (at(e) >= hidden) continue;
+                NormFour<float> t;
+#pragma unroll
+                for (int u = 0; u < 4; ++u) t.v[u] = xv[e][u];
+                *reinterpret_cast<NormFour<float>*>(x + base + at(e)) = t;
+            }
+        }
+    }
+    if (!out) return;
+    if (CONV) {
+        // (a thread's own columns of the carried rows: each moves up by one as it is read)
+        const int taps = conv.taps;
+#pragma unroll
+        for (int e = 0; e < G; ++e) {
+            const int i = at(e);
+            if (i >= hidden) continue;
+            NormFour<float> now, acc;
+#pragma unroll
+            for (int u = 0; u < 4; ++u) now.v[u] = acc.v[u] = xv[e][u];
+            auto tap = [&](const NormFour<float>& wv, const NormFour<float>& v) {
+#pragma unroll
+                for (int u = 0; u < 4; ++u) acc.v[u] = fmaf(wv.v[u], v.v[u], acc.v[u]);
+            };
+#pragma unroll
+            for (int k = 0; k < kHeldTaps; ++k) {
+                if (k + 1 < taps) {
+                    tap(held_w[e][k], held_c[e][k]);
+                    if (k > 0) carry_four(k - 1, i, held_c[e][k]);
+                } else if (k + 1 == taps) {
+                    tap(held_w[e][k], now);
+                }
+            }
+            for (int k = kHeldTaps; k < taps; ++k) {
+                const NormFour<float> wv = *reinterpret_cast<const NormFour<float>*>(conv.weight + static_cast<size_t>(k) * hidden + i);
+                if (k + 1 < taps) {
+                    const NormFour<float> v = carried_four(k, i);
+                    tap(wv, v);
+                    carry_four(k - 1, i, v);
+                } else {
+                    tap(wv, now);
+                }
+            }
+            if (taps > 1) carry_four(taps - 2, i, now);
+            NormFour<TO> t;
+#pragma unroll
+            for (int u = 0; u < 4; ++u) t.v[u] = from_float<TO>(acc.v[u]);
+            *reinterpret_cast<NormFour<TO>*>(out + static_cast<size_t>(orow) * hidden + i) = t;
+        }
+        return;
+    }
+    held_stats<G>(xv, hidden, o_kind, o_eps, scratch, mean, inv);
+    TO* o = out + static_cast<size_t>(orow) * hidden;
+#pragma unroll
+    for (int e = 0; e < G; ++e) {
+        if (at(e) >= hidden) continue;
+        NormFour<TO> t;
+#pragma unroll
+        for (int u = 0; u < 4; ++u)
+            t.v[u] = from_float<TO>(o_kind != kNormNone ? (xv[e][u] - mean) * inv * (o_offset + w[e][u]) : xv[e][u]);
+        *reinterpret_cast<NormFour<TO>*>(o + at(e)) = t;
+    }
+}
+
 // delta_type / out_type: 0 float32, 1 bfloat16.  Returns 0, a HIP error code, or -1 for sizes it does not take.
 WLLM_API int wllm_norm_add(float* x, const void* delta, int delta_type, int splits, long long split_stride, int d_kind,
                            const float* d_weight, float d_eps, float d_offset, const int* rows, void* out, int out_type,
@@ -203,6 +433,35 @@ WLLM_API int wllm_norm_add(float* x, const void* delta, int delta_type, int spli
     if (delta && d_kind != kNormNone && !d_weight) return -1;
     if (out && o_kind != kNormNone && !o_weight) return -1;
     if (!delta && !out) return 0;
+    auto aligned = [](const void* p, size_t bytes) { return reinterpret_cast<uintptr_t>(p) % bytes == 0; };
+    const bool four = hidden % 4 == 0 && hidden <= 4096 * 4 && (splits <= 1 || split_stride % 4 == 0) &&
+                      (!extra || extra_splits <= 1 || extra_stride % 4 == 0) && aligned(x, 16) && aligned(delta, 16) && aligned(out, 16) &&
+                      aligned(extra, 16) && aligned(d_weight, 16) && aligned(o_weight, 16) && aligned(s_weight, 16) && aligned(conv_weight, 16);
+    const int conv_aligned = conv_state_stride % 4 == 0 && conv_carried_offset % 4 == 0 && aligned(conv_state, 16);
+    if (four) {
+        // many rows: groups of four a thread so that some workgroups share a compute unit; few rows: one, so that a row's
+        // loads are all on their way at once
+        const int quads = hidden / 4;
+        const int groups = quads > 2048 ? 4 : quads > 1024 ? 2 : num_rows <= 256 || quads <= 256 ? 1 : 2;
+        const int four_threads = ((quads + groups - 1) / groups + 63) / 64 * 64;
+#define LAUNCH_C(TD, TO, G, CONV)                                                                                      \
+    norm_add_four_kernel<TD, TO, G, CONV><<<num_rows, four_threads, 0, stream>>>(                                      \
+        x, static_cast<const TD*>(delta), splits, static_cast<size_t>(split_stride), d_kind, d_weight, d_eps, d_offset, rows, \
+        static_cast<TO*>(out), o_kind, o_weight, o_eps, o_offset, hidden, join, conv, conv_aligned)
+#define LAUNCH_G(TD, TO, G) do { if (conv_weight) LAUNCH_C(TD, TO, G, true); else LAUNCH_C(TD, TO, G, false); } while (0)
+#define LAUNCH(TD, TO)                          \
+    if (groups == 1) LAUNCH_G(TD, TO, 1);       \
+    else if (groups == 2) LAUNCH_G(TD, TO, 2);  \
+    else LAUNCH_G(TD, TO, 4)
+        if (delta_type && out_type) { LAUNCH(bf16, bf16); }
+        else if (delta_type) { LAUNCH(bf16, float); }
+        else if (out_type) { LAUNCH(float, bf16); }
+        else { LAUNCH(float, float); }
+#undef LAUNCH
+#undef LAUNCH_G
+#undef LAUNCH_C
+        return launch_status();
+    }
     const size_t smem = sizeof(float) * static_cast<size_t>(hidden);
     // The few rows of a decode step: a row's time is that of its chain of trips to memory (a stack of partial
     // sums to add, the stream, the weights), so as many threads as give each two elements; many rows: 256.
