@@ -357,6 +357,45 @@ def test_a_batch_of_unequal_requests_against_each_alone(H, G, d, dv, taps, chunk
     assert torch.equal(together[4], state0[4])
 
 
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("H,G,d,dv,taps", [(16, 2, 128, 128, 4), (16, 4, 96, 160, 3), (8, 4, 192, 256, 4), (16, 2, 128, 128, 1), (16, 2, 128, 132, 6)])
+def test_the_inputs_of_many_tokens_are_those_of_few(H, G, d, dv, taps, dtype):
+    """A step of some thousand tokens (several a wavefront, their inputs asked for together where they are of one portion)
+    against the same requests 50 tokens at a time: the same bits, whatever borders fall among a wavefront's tokens."""
+    g = torch.Generator().manual_seed(d + taps)
+    lengths = [2, 1, 1001, 5, 3, 1, 1, 4, 766, 7, 6, 2, 503]
+    n, channels, count = sum(lengths), 2 * G * d + H * dv, len(lengths)
+    dp, memory = ops.delta_padded(d), ops.delta_state_size(H, d, dv)
+    total = -(-(memory + (taps - 1) * channels) // 4) * 4
+    x = torch.randn(n, channels, generator=g).to(DEV, dtype)
+    z, b = torch.randn(n, H * d, generator=g).to(DEV, dtype), torch.randn(n, H, generator=g).to(DEV, dtype)
+    conv, rate = torch.randn(taps, channels, generator=g).to(DEV), (torch.rand(H, generator=g) + 0.1).to(DEV)
+    bias = (-3.0 + torch.randn(H * d, generator=g)).to(DEV)
+    state0 = torch.randn(count, total, generator=g).to(DEV)
+
+    def run(x, z, b, lengths, slots, state):
+        m = x.shape[0]
+        start = torch.cumsum(torch.tensor([0] + lengths), 0)[:-1].tolist()
+        of = torch.repeat_interleave(torch.arange(len(lengths), dtype=torch.int32), torch.tensor(lengths)).to(DEV)
+        nan = lambda *s: torch.full(s, float("nan"), device=DEV)
+        out = nan(2, m, G * dp), nan(m, G), nan(m, H * dv).to(dtype), nan(m, H * dp), nan(m, H)
+        ops.delta_inputs(x, z, b, conv, rate, bias, state, memory, of, _i32(start), _i32(lengths), _i32(slots), *out, q_scale=d ** -0.5,
+                         unit_eps=1e-6, single_tokens=False, heads=H, groups=G, head_dim=d, value_dim=dv)
+        return out
+
+    together, apart = state0.clone(), state0.clone()
+    all_at_once = run(x, z, b, lengths, list(range(count)), together)
+    at = 0
+    for slot, length in enumerate(lengths):
+        for lo in range(at, at + length, 50):
+            part = slice(lo, min(lo + 50, at + length))
+            few = run(x[part], z[part], b[part], [part.stop - lo], [slot], apart)
+            for name, one, other in zip(("qk", "kq", "v", "f", "beta"), all_at_once, few):
+                assert torch.equal(one[:, part] if name == "qk" else one[part], other), f"{name}, request {slot}, tokens from {lo - at}"
+        at += length
+    assert torch.equal(together, apart)
+
+
 # ---- the engine -----------------------------------------------------------------------------------------
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("family", list(FAMILIES))

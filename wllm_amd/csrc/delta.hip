@@ -132,36 +132,66 @@ delta_inputs_kernel(const T* __restrict__ xqkv, long long x_stride, const T* __r
 }
 
 // The same with four consecutive channels a lane (D, P, the rows' strides and the carried rows' place are multiples of
-// four): lanes 0 .. 31 of a group's wavefront hold q, lanes 32 .. 63 k.
+// four): lanes 0 .. 31 of a group's wavefront hold q, lanes 32 .. 63 k.  Many tokens: a wavefront takes GROUP tokens and keeps what
+// they share in registers: up to four taps a channel, the decays' biases and, where the tokens and the inputs before them are
+// all of one portion, the inputs, each of them asked for once and all of them before the first is waited for.
 template <typename T> struct alignas(4 * sizeof(T)) DeltaFour { T v[4]; };
+
+template <typename T>
+__device__ __forceinline__ float4 four_floats(const T* p) {
+    const DeltaFour<T> e = *reinterpret_cast<const DeltaFour<T>*>(p);
+    return make_float4(to_float(e.v[0]), to_float(e.v[1]), to_float(e.v[2]), to_float(e.v[3]));
+}
+// Four elements as they lie in memory, and N of them in registers before the next statement (a compiler left alone asks
+// for each where it is used and waits for every one).
+template <typename T>
+using RawFour = int __attribute__((ext_vector_type(sizeof(T))));
+template <typename R, int N>
+__device__ __forceinline__ void all_there(R (&x)[N]) {
+#pragma unroll
+    for (int i = 0; i < N; ++i) asm volatile("" : "+v"(x[i]));
+}
+template <typename T>
+__device__ __forceinline__ float4 four_floats(const RawFour<T> raw) {
+    const DeltaFour<T> e = __builtin_bit_cast(DeltaFour<T>, raw);
+    return make_float4(to_float(e.v[0]), to_float(e.v[1]), to_float(e.v[2]), to_float(e.v[3]));
+}
+__device__ __forceinline__ float dot4(const float4 a, const float4 b) { return fmaf(a.w, b.w, fmaf(a.z, b.z, fmaf(a.y, b.y, a.x * b.x))); }
+
+constexpr int kHeldTaps = 4;
+constexpr int kDeltaGroup = 4;                  // tokens a wavefront, where there are many (eight: the last wavefronts wait)
+struct HeldTaps {
+    float4 w[kHeldTaps];                         // the first ones
+    __device__ __forceinline__ void load(const float* from, int channels, int taps, int c) {
+#pragma unroll
+        for (int k = 0; k < kHeldTaps; ++k)
+            w[k] = k < taps ? *reinterpret_cast<const float4*>(from + static_cast<size_t>(k) * channels + c) : make_float4(0.f, 0.f, 0.f, 0.f);
+    }
+};
 
 template <typename T, bool CARRY>
 __device__ __forceinline__ float4 short_conv_four(const T* now, long long stride, int local, float* carried, const float* w,
-                                                  int channels, int taps, int c) {
-    const DeltaFour<T> mine = *reinterpret_cast<const DeltaFour<T>*>(now + c);
+                                                  const HeldTaps& held, int channels, int taps, int c) {
     float4 acc = make_float4(0.f, 0.f, 0.f, 0.f);
-    auto add = [&](const float4 wv, const float4 x) {
+    auto tap = [&](int k, const float4 wv) {
+        const int back = taps - 1 - k;           // how many tokens ago
+        float4 x;
+        if (back > 0 && (CARRY || local < back)) {
+            x = *reinterpret_cast<const float4*>(carried + static_cast<size_t>(k + (CARRY ? 0 : local)) * channels + c);
+            if (CARRY && k > 0) *reinterpret_cast<float4*>(carried + static_cast<size_t>(k - 1) * channels + c) = x;
+        } else {
+            x = four_floats(now + c - back * stride);
+            if (CARRY && taps > 1) *reinterpret_cast<float4*>(carried + static_cast<size_t>(taps - 2) * channels + c) = x;
+        }
         acc.x = fmaf(wv.x, x.x, acc.x);
         acc.y = fmaf(wv.y, x.y, acc.y);
         acc.z = fmaf(wv.z, x.z, acc.z);
         acc.w = fmaf(wv.w, x.w, acc.w);
     };
-#pragma unroll 4
-    for (int k = 0; k + 1 < taps; ++k) {
-        const int back = taps - 1 - k;
-        float4 x;
-        if (CARRY || local < back) {
-            x = *reinterpret_cast<const float4*>(carried + static_cast<size_t>(k + (CARRY ? 0 : local)) * channels + c);
-            if (CARRY && k > 0) *reinterpret_cast<float4*>(carried + static_cast<size_t>(k - 1) * channels + c) = x;
-        } else {
-            const DeltaFour<T> e = *reinterpret_cast<const DeltaFour<T>*>(now + c - back * stride);
-            x = make_float4(to_float(e.v[0]), to_float(e.v[1]), to_float(e.v[2]), to_float(e.v[3]));
-        }
-        add(*reinterpret_cast<const float4*>(w + static_cast<size_t>(k) * channels + c), x);
-    }
-    const float4 x = make_float4(to_float(mine.v[0]), to_float(mine.v[1]), to_float(mine.v[2]), to_float(mine.v[3]));
-    if (CARRY && taps > 1) *reinterpret_cast<float4*>(carried + static_cast<size_t>(taps - 2) * channels + c) = x;
-    add(*reinterpret_cast<const float4*>(w + static_cast<size_t>(taps - 1) * channels + c), x);
+#pragma unroll
+    for (int k = 0; k < kHeldTaps; ++k)
+        if (k < taps) tap(k, held.w[k]);
+    for (int k = kHeldTaps; k < taps; ++k) tap(k, *reinterpret_cast<const float4*>(w + static_cast<size_t>(k) * channels + c));
     acc.x /= 1.f + expf(-acc.x);
     acc.y /= 1.f + expf(-acc.y);
     acc.z /= 1.f + expf(-acc.z);
@@ -169,88 +199,170 @@ __device__ __forceinline__ float4 short_conv_four(const T* now, long long stride
     return acc;
 }
 
-__device__ __forceinline__ float dot4(const float4 a, const float4 b) { return fmaf(a.w, b.w, fmaf(a.z, b.z, fmaf(a.y, b.y, a.x * b.x))); }
+// The inputs of GROUP tokens and of the taps - 1 <= kHeldTaps - 1 before them, and the convolution of the token at place g.
+// (what stands behind the last row is a copy of it; held taps beyond the last one are zeros)
+template <typename T, int GROUP>
+struct ConvWindow {
+    RawFour<T> x[GROUP + kHeldTaps - 1];
+    __device__ __forceinline__ void load(const T* xqkv, long long stride, int first, int last, int taps, int c) {
+        const T* from = xqkv + static_cast<long long>(first - (taps - 1)) * stride + c;
+        const int rows = last - first + taps - 1;
+#pragma unroll
+        for (int r = 0; r < GROUP + kHeldTaps - 1; ++r)
+            x[r] = *reinterpret_cast<const RawFour<T>*>(from + static_cast<long long>(min(r, rows - 1)) * stride);
+        all_there(x);
+    }
+    __device__ __forceinline__ float4 at(int g, const HeldTaps& held) const {
+        float4 acc = make_float4(0.f, 0.f, 0.f, 0.f);
+#pragma unroll
+        for (int k = 0; k < kHeldTaps; ++k) {
+            const float4 in = four_floats<T>(x[g + k]);
+            acc.x = fmaf(held.w[k].x, in.x, acc.x);
+            acc.y = fmaf(held.w[k].y, in.y, acc.y);
+            acc.z = fmaf(held.w[k].z, in.z, acc.z);
+            acc.w = fmaf(held.w[k].w, in.w, acc.w);
+        }
+        acc.x /= 1.f + expf(-acc.x);
+        acc.y /= 1.f + expf(-acc.y);
+        acc.z /= 1.f + expf(-acc.z);
+        acc.w /= 1.f + expf(-acc.w);
+        return acc;
+    }
+};
 
-template <typename T, bool CARRY>
+template <typename T, bool CARRY, int GROUP, int PER>
 __global__ void __launch_bounds__(kWave * kDeltaWaves)
 delta_inputs_four_kernel(const T* __restrict__ xqkv, long long x_stride, const T* __restrict__ z, long long z_stride,
                          const T* __restrict__ b, long long b_stride, T* __restrict__ v, DeltaInputs a) {
-    const int token = blockIdx.x;
+    const int first = blockIdx.x * GROUP, last = min(a.tokens, first + GROUP);
     const int lane = threadIdx.x % kWave, wave = threadIdx.x / kWave;
-    const int seg = a.token_segment[token];
-    const int local = token - a.seg_q_start[seg];
     const int channels = 2 * a.groups * a.d + a.heads * a.p_dim;
-    float* carried = a.state + static_cast<size_t>(a.state_slots[seg]) * a.state_stride + a.carried_offset;
-    const T* xt = xqkv + static_cast<size_t>(token) * x_stride;
-    auto convolved = [&](int c) { return short_conv_four<T, CARRY>(xt, x_stride, local, carried, a.conv_w, channels, a.taps, c); };
-    int unit = blockIdx.y * kDeltaWaves + wave;
+    const int unit = blockIdx.y * kDeltaWaves + wave;
+    // (a token's place in its segment and its request's carried rows)
+    auto convolved = [&](int token, const HeldTaps& held, int c) {
+        const int seg = a.token_segment[token];
+        float* carried = a.state + static_cast<size_t>(a.state_slots[seg]) * a.state_stride + a.carried_offset;
+        return short_conv_four<T, CARRY>(xqkv + static_cast<size_t>(token) * x_stride, x_stride, token - a.seg_q_start[seg], carried,
+                                         a.conv_w, held, channels, a.taps, c);
+    };
+    bool inside = false;                         // the window of all the tokens lies in one portion
+    if (GROUP > 1 && a.taps <= kHeldTaps) {
+        const int seg = a.token_segment[first];
+        inside = seg == a.token_segment[last - 1] && first - a.seg_q_start[seg] >= a.taps - 1;
+    }
     if (unit < a.groups) {
-        constexpr int kPer = 2;                  // heads of up to 32 * 4 * 2 channels
         const int half = lane / 32;              // 0: q, 1: k
-        float4 x[kPer];
-        float ss = 0.f;
+        HeldTaps held[PER];
 #pragma unroll
-        for (int j = 0; j < kPer; ++j) {
+        for (int j = 0; j < PER; ++j) {
             const int i = 4 * (lane % 32 + 32 * j);
-            x[j] = make_float4(0.f, 0.f, 0.f, 0.f);
-            if (i < a.d) x[j] = convolved((half * a.groups + unit) * a.d + i);
-            ss += dot4(x[j], x[j]);
+            held[j].load(a.conv_w, channels, i < a.d ? a.taps : 0, (half * a.groups + unit) * a.d + i);
         }
-        ss = row_halves_sum(ss);
-        const float inv = (half ? 1.f : a.q_scale) / sqrtf(ss + a.unit_eps);
-        float* out = a.qk + (static_cast<size_t>(half) * a.tokens + token) * a.groups * a.dp + static_cast<size_t>(unit) * a.dp;
-        float dot = 0.f;
+        auto finish = [&](int token, float4 (&x)[PER]) {
+            float ss = 0.f;
 #pragma unroll
-        for (int j = 0; j < kPer; ++j) {
-            const int i = 4 * (lane % 32 + 32 * j);
-            x[j].x *= inv;
-            x[j].y *= inv;
-            x[j].z *= inv;
-            x[j].w *= inv;
-            const float4 other = make_float4(from_other_half(x[j].x), from_other_half(x[j].y), from_other_half(x[j].z),
-                                             from_other_half(x[j].w));
-            dot += dot4(x[j], other);
-            if (i < a.d) *reinterpret_cast<float4*>(out + i) = x[j];
+            for (int j = 0; j < PER; ++j) ss += dot4(x[j], x[j]);
+            ss = row_halves_sum(ss);
+            const float inv = (half ? 1.f : a.q_scale) / sqrtf(ss + a.unit_eps);
+            float* out = a.qk + (static_cast<size_t>(half) * a.tokens + token) * a.groups * a.dp + static_cast<size_t>(unit) * a.dp;
+            float dot = 0.f;
+#pragma unroll
+            for (int j = 0; j < PER; ++j) {
+                const int i = 4 * (lane % 32 + 32 * j);
+                x[j].x *= inv;
+                x[j].y *= inv;
+                x[j].z *= inv;
+                x[j].w *= inv;
+                const float4 other = make_float4(from_other_half(x[j].x), from_other_half(x[j].y), from_other_half(x[j].z),
+                                                 from_other_half(x[j].w));
+                dot += dot4(x[j], other);
+                if (i < a.d) *reinterpret_cast<float4*>(out + i) = x[j];
+            }
+            dot = row_halves_sum(dot);
+            if (lane == 0) a.kq[static_cast<size_t>(token) * a.groups + unit] = dot;
+        };
+        if (GROUP > 1 && inside) {
+            ConvWindow<T, GROUP> window[PER];
+#pragma unroll
+            for (int j = 0; j < PER; ++j)        // (a lane beyond the head reads its last channels: its taps are zeros)
+                window[j].load(xqkv, x_stride, first, last, a.taps, (half * a.groups + unit) * a.d + min(4 * (lane % 32 + 32 * j), a.d - 4));
+#pragma unroll
+            for (int g = 0; g < GROUP; ++g) {
+                if (first + g >= last) break;
+                float4 x[PER];
+#pragma unroll
+                for (int j = 0; j < PER; ++j) x[j] = window[j].at(g, held[j]);
+                finish(first + g, x);
+            }
+            return;
         }
-        dot = row_halves_sum(dot);
-        if (lane == 0) a.kq[static_cast<size_t>(token) * a.groups + unit] = dot;
+        for (int token = first; token < last; ++token) {
+            float4 x[PER];
+#pragma unroll
+            for (int j = 0; j < PER; ++j) {
+                const int i = 4 * (lane % 32 + 32 * j);
+                x[j] = make_float4(0.f, 0.f, 0.f, 0.f);
+                if (i < a.d) x[j] = convolved(token, held[j], (half * a.groups + unit) * a.d + i);
+            }
+            finish(token, x);
+        }
         return;
     }
-    unit -= a.groups;
     const int v_width = a.heads * a.p_dim, f_width = a.heads * a.d;
-#pragma unroll
-    for (int j = 0; j < kDeltaPer; ++j) {
-        int e = (unit * kWave * kDeltaPer + kWave * j + lane) * 4;
-        if (e < v_width) {
-            const float4 x = convolved(2 * a.groups * a.d + e);
+    int e = ((unit - a.groups) * kWave + lane) * 4;
+    if (e < v_width) {
+        const int c = 2 * a.groups * a.d + e;
+        HeldTaps held;
+        held.load(a.conv_w, channels, a.taps, c);
+        auto write = [&](int token, const float4 x) {
             DeltaFour<T> r;
             r.v[0] = from_float<T>(x.x);
             r.v[1] = from_float<T>(x.y);
             r.v[2] = from_float<T>(x.z);
             r.v[3] = from_float<T>(x.w);
             *reinterpret_cast<DeltaFour<T>*>(v + static_cast<size_t>(token) * v_width + e) = r;
-            continue;
+        };
+        if (GROUP > 1 && inside) {
+            ConvWindow<T, GROUP> window;
+            window.load(xqkv, x_stride, first, last, a.taps, c);
+#pragma unroll
+            for (int g = 0; g < GROUP; ++g)
+                if (first + g < last) write(first + g, window.at(g, held));
+            return;
         }
-        e -= v_width;
-        if (e < f_width) {
-            const float rate = a.rate[e / a.d];
-            const DeltaFour<T> zv = *reinterpret_cast<const DeltaFour<T>*>(z + static_cast<size_t>(token) * z_stride + e);
-            const float4 bias = *reinterpret_cast<const float4*>(a.dt_bias + e);
+        for (int token = first; token < last; ++token) write(token, convolved(token, held, c));
+        return;
+    }
+    e -= v_width;
+    if (e < f_width) {
+        const float rate = a.rate[e / a.d];
+        const float4 bias = *reinterpret_cast<const float4*>(a.dt_bias + e);
+        RawFour<T> held[GROUP];
+#pragma unroll
+        for (int g = 0; g < GROUP; ++g)
+            held[g] = *reinterpret_cast<const RawFour<T>*>(z + static_cast<size_t>(min(first + g, last - 1)) * z_stride + e);
+        all_there(held);
+#pragma unroll
+        for (int g = 0; g < GROUP; ++g) {
+            const int token = first + g;
+            if (token >= last) break;
+            const float4 zv = four_floats<T>(held[g]);
             float4 r;
-            r.x = expf(-rate * delta_softplus(to_float(zv.v[0]) + bias.x));
-            r.y = expf(-rate * delta_softplus(to_float(zv.v[1]) + bias.y));
-            r.z = expf(-rate * delta_softplus(to_float(zv.v[2]) + bias.z));
-            r.w = expf(-rate * delta_softplus(to_float(zv.v[3]) + bias.w));
+            r.x = expf(-rate * delta_softplus(zv.x + bias.x));
+            r.y = expf(-rate * delta_softplus(zv.y + bias.y));
+            r.z = expf(-rate * delta_softplus(zv.z + bias.z));
+            r.w = expf(-rate * delta_softplus(zv.w + bias.w));
             *reinterpret_cast<float4*>(a.f + static_cast<size_t>(token) * f_width + e) = r;
-            continue;
         }
-        e -= f_width;
+        return;
+    }
+    e -= f_width;
+    for (int token = first; token < last; ++token)
 #pragma unroll
         for (int u = 0; u < 4; ++u)
             if (e + u < a.heads)
                 a.beta[static_cast<size_t>(token) * a.heads + e + u] =
                     1.f / (1.f + expf(-to_float(b[static_cast<size_t>(token) * b_stride + e + u])));
-    }
 }
 
 WLLM_API int wllm_delta_inputs(const void* xqkv, long long x_stride, const void* z, long long z_stride, const void* b,
@@ -278,23 +390,29 @@ WLLM_API int wllm_delta_inputs(const void* xqkv, long long x_stride, const void*
                       reinterpret_cast<uintptr_t>(f) % 16 == 0;
     if (four) {
         const long long fours = rest / 4 + 1;    // (beta's last four may be partly there)
-        const long long four_units = groups + (fours + kWave * kDeltaPer - 1) / (kWave * kDeltaPer);
-        const dim3 four_grid(tokens, static_cast<unsigned>((four_units + kDeltaWaves - 1) / kDeltaWaves));
-#define LAUNCH(T, CARRY)                                                                                                \
-    delta_inputs_four_kernel<T, CARRY><<<four_grid, kWave * kDeltaWaves, 0, stream>>>(                                  \
-        static_cast<const T*>(xqkv), x_stride, static_cast<const T*>(z), z_stride, static_cast<const T*>(b), b_stride,  \
-        static_cast<T*>(v), a)
-        if (is_bf16) { if (single_tokens) LAUNCH(bf16, true); else LAUNCH(bf16, false); }
-        else { if (single_tokens) LAUNCH(float, true); else LAUNCH(float, false); }
+        const long long four_units = groups + (fours + kWave - 1) / kWave;
+        const unsigned four_pieces = static_cast<unsigned>((four_units + kDeltaWaves - 1) / kDeltaWaves);
+        // (about eight wavefronts a SIMD remain with four tokens each)
+        const bool many = !single_tokens && static_cast<long long>(tokens) * four_pieces >= 8192;
+#define LAUNCH(T, CARRY, GROUP, PER)                                                                                    \
+    delta_inputs_four_kernel<T, CARRY, GROUP, PER>                                                                      \
+        <<<dim3((tokens + GROUP - 1) / GROUP, four_pieces), kWave * kDeltaWaves, 0, stream>>>(                          \
+            static_cast<const T*>(xqkv), x_stride, static_cast<const T*>(z), z_stride, static_cast<const T*>(b), b_stride, \
+            static_cast<T*>(v), a)
+#define BY_TOKENS(T, PER)                                                                                               \
+    if (single_tokens) LAUNCH(T, true, 1, PER); else if (many) LAUNCH(T, false, kDeltaGroup, PER); else LAUNCH(T, false, 1, PER)
+        if (is_bf16) { if (d <= 128) { BY_TOKENS(bf16, 1); } else { BY_TOKENS(bf16, 2); } }
+        else { if (d <= 128) { BY_TOKENS(float, 1); } else { BY_TOKENS(float, 2); } }
+#undef BY_TOKENS
 #undef LAUNCH
     } else {
-    const dim3 grid(tokens, static_cast<unsigned>(pieces));
+        const dim3 grid(tokens, static_cast<unsigned>(pieces));
 #define LAUNCH(T, CARRY)                                                                                                \
-    delta_inputs_kernel<T, CARRY><<<grid, kWave * kDeltaWaves, 0, stream>>>(                                            \
-        static_cast<const T*>(xqkv), x_stride, static_cast<const T*>(z), z_stride, static_cast<const T*>(b), b_stride,  \
-        static_cast<T*>(v), a)
-    if (is_bf16) { if (single_tokens) LAUNCH(bf16, true); else LAUNCH(bf16, false); }
-    else { if (single_tokens) LAUNCH(float, true); else LAUNCH(float, false); }
+        delta_inputs_kernel<T, CARRY><<<grid, kWave * kDeltaWaves, 0, stream>>>(                                        \
+            static_cast<const T*>(xqkv), x_stride, static_cast<const T*>(z), z_stride, static_cast<const T*>(b), b_stride,\
+            static_cast<T*>(v), a)
+        if (is_bf16) { if (single_tokens) LAUNCH(bf16, true); else LAUNCH(bf16, false); }
+        else { if (single_tokens) LAUNCH(float, true); else LAUNCH(float, false); }
 #undef LAUNCH
     }
     if (const int err = launch_status()) return err;
